@@ -6,7 +6,10 @@ registry, host-only) by the host compiler against the installed torch headers, a
 linked into one shared object loaded with `torch.ops.load_library`. The `.so` lives next to this
 file so it travels with the repository snapshot to the GPU box.
 
-    python -m distributed_llm_alignment_amd._build [--force] [-j N] [--sanitize address,undefined]
+Sources form groups, one library each: `core` (csrc/*, `_C.so`) and `mix` (csrc/mix/*, `_C_mix.so`:
+the kernels of per-layer designs). A program that needs one group builds and loads that one alone.
+
+    python -m distributed_llm_alignment_amd._build [--group core|mix] [--force] [-j N] [--sanitize address,undefined]
 
 `--sanitize` (or DLA_SANITIZE=address,undefined) builds a host-sanitized variant into a separate
 `_C_san.so` (select it with DLA_EXT_PATH=.../_C_san.so): the launchers, torch bindings and
@@ -28,9 +31,12 @@ from pathlib import Path
 PKG_DIR = Path(__file__).resolve().parent
 CSRC = PKG_DIR / "csrc"
 OUT_SO = PKG_DIR / "_C.so"
+GROUPS = {"core": (CSRC, OUT_SO), "mix": (CSRC / "mix", PKG_DIR / "_C_mix.so")}
 SAN_SO = PKG_DIR / "_C_san.so"
 OBJ_DIR = PKG_DIR.parent / "build" / "dla_objs"
 ARCH = os.environ.get("DLA_OFFLOAD_ARCH", "gfx950")
+# no v_pk_{add,mul,fma}_f32: some forms of the packed fp32 instructions gave wrong results now and then
+NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 ROCM = Path(os.environ.get("ROCM_PATH", "/opt/rocm"))
 
 
@@ -49,13 +55,14 @@ def _hipcc() -> str:
     return str(cand) if cand.exists() else "hipcc"
 
 
-def _sources():
-    hips = sorted(CSRC.glob("*.hip"))
-    return hips, sorted(CSRC.glob("*.cpp"))
+def _sources(group: str = "core"):
+    d = GROUPS[group][0]
+    return sorted(d.glob("*.hip")), sorted(d.glob("*.cpp"))
 
 
-def _headers():
-    return sorted(CSRC.glob("*.h"))
+def _headers(group: str = "core"):
+    own = [] if group == "core" else sorted(GROUPS[group][0].glob("*.h"))
+    return sorted(CSRC.glob("*.h")) + own
 
 
 def _newer(src: Path, dst: Path, deps) -> bool:
@@ -83,13 +90,15 @@ def _san_list(sanitize) -> list:
 
 
 def build(force: bool = False, jobs: int | None = None, verbose: bool = False,
-          sanitize: str | None = None) -> Path:
-    """Compile every HIP kernel for gfx950 and link `_C.so` (or the host-sanitized `_C_san.so`).
-    Returns the .so path."""
+          sanitize: str | None = None, group: str = "core") -> Path:
+    """Compile the HIP kernels of one group for gfx950 and link its library (or, core only, the
+    host-sanitized `_C_san.so`). Returns the .so path."""
     inc, lib, abi = _torch_paths()
     san = _san_list(sanitize if sanitize is not None else os.environ.get("DLA_SANITIZE_BUILD"))
-    obj_dir = OBJ_DIR.parent / "dla_objs_san" if san else OBJ_DIR
-    out_so = SAN_SO if san else OUT_SO
+    if san and group != "core":
+        raise ValueError("host sanitizers: core group only")
+    obj_dir = OBJ_DIR.parent / "dla_objs_san" if san else OBJ_DIR if group == "core" else OBJ_DIR / group
+    out_so = SAN_SO if san else GROUPS[group][1]
     obj_dir.mkdir(parents=True, exist_ok=True)
     hsan = [f"-Xarch_host -fsanitize={x}".split() for x in san]
     # vptr checks need the clang UBSan C++ runtime, which the g++-built bindings do not link; so
@@ -99,8 +108,8 @@ def build(force: bool = False, jobs: int | None = None, verbose: bool = False,
     hextra = ["-fno-sanitize=function"] if "undefined" in san else []
     hsan = [a for pair in hsan for a in pair] + [a for x in extra + hextra for a in ("-Xarch_host", x)] if san else []
     gsan = [f"-fsanitize={x}" for x in san] + extra if san else []
-    hips, bindings = _sources()
-    headers = _headers()
+    hips, bindings = _sources(group)
+    headers = _headers(group)
     jobs = jobs or min(8, os.cpu_count() or 4)
     hipcc = _hipcc()
     common = ["-O3", "-std=c++17", "-fPIC", f"-I{CSRC}"]
@@ -110,7 +119,7 @@ def build(force: bool = False, jobs: int | None = None, verbose: bool = False,
         obj = obj_dir / (src.stem + ".o")
         objs.append(obj)
         if force or _newer(src, obj, headers):
-            tasks.append([hipcc, f"--offload-arch={ARCH}", "-munsafe-fp-atomics", *common, *hsan,
+            tasks.append([hipcc, f"--offload-arch={ARCH}", "-munsafe-fp-atomics", *NO_PACKED_FP32, *common, *hsan,
                           "-c", str(src), "-o", str(obj)])
     cxx = shutil.which("g++") or shutil.which("c++") or "c++"
     py_inc = sysconfig.get_paths()["include"]
@@ -136,15 +145,20 @@ def build(force: bool = False, jobs: int | None = None, verbose: bool = False,
     return out_so
 
 
+def build_all(force: bool = False, jobs: int | None = None, verbose: bool = False) -> list:
+    return [build(force=force, jobs=jobs, verbose=verbose, group=g) for g in GROUPS]
+
+
 def main(argv=None) -> int:
     ap = argparse.ArgumentParser(description=__doc__)
     ap.add_argument("--force", action="store_true")
     ap.add_argument("-j", "--jobs", type=int, default=None)
     ap.add_argument("-v", "--verbose", action="store_true")
     ap.add_argument("--sanitize", default=None, help="host sanitizers, e.g. address,undefined")
+    ap.add_argument("--group", choices=sorted(GROUPS), default=None, help="one group (default: all)")
     a = ap.parse_args(argv)
-    so = build(force=a.force, jobs=a.jobs, verbose=a.verbose, sanitize=a.sanitize)
-    print(f"built {so}")
+    for group in [a.group] if a.group else ["core"] if a.sanitize else list(GROUPS):
+        print(f"built {build(force=a.force, jobs=a.jobs, verbose=a.verbose, sanitize=a.sanitize, group=group)}")
     return 0
 
 

@@ -1,0 +1,50 @@
+// Host/device parameter blocks of the mixer kernels (latent attention, retention).
+#pragma once
+#include <cstdint>
+
+namespace dla {
+
+struct RetentionParams {
+  const void* qkvg;       // [B, T, H (2 dim + 2 vdim)] rows [q | k | v | g], row stride ld, contiguous in T
+  int64_t ld;
+  void* y;                // [B, T, H vdim]
+  float* state;           // [B, H, vdim, dim]
+  float* work;            // chunked form: [B, H, nc, vdim, dim]
+  const float* decay;     // [2, H]: decay, log2 decay
+  const float* cos_t;     // [positions, rot / 2]
+  const float* sin_t;
+  const int64_t* slot;    // column of the first token on the device (nullptr: base)
+  const int* kv_start;    // [B] first real column, or nullptr
+  int64_t base;           // column of the first token
+  int B, T, H, dim, vdim, rot;
+  float eps, kscale;
+  int chunk, nc;
+  int npos;               // rows of the rotary tables
+  int fresh;              // the state starts at zero (base == 0)
+};
+
+struct LatentParams {
+  const void* q;          // [B, T, H (dim + rot)], contiguous
+  const void* kv;         // prefill: [B, S, H (dim + vdim)] = [keys | values], contiguous
+  const void* kr;         // prefill: rotated key part, [B, S, rot] inside cache rows
+  int64_t kr_sb, kr_st;   // its strides
+  const void* latent;     // decode: cache [B, Tmax, R + rot]
+  int64_t l_sb, l_st;
+  const void* kv_up;      // decode: [H (dim + vdim), R]
+  void* qcat;             // decode: [B, H, R + rot] query in latent space | rotated part
+  void* o;                // [B, T, H vdim]
+  float* part_o;          // decode: [B, H, ns, R]
+  float* part_ml;         // decode: [B, H, ns, 2]
+  const float* cos_t;
+  const float* sin_t;
+  const int64_t* slot;    // decode: column of the newest token
+  const int* kv_start;    // [B] first real column, or nullptr
+  int B, T, S, H, dim, rot, vdim, R;
+  int q_base, k_base;     // prefill: column of query 0 / key 0
+  int window;             // 0: none
+  float scale;
+  int ns;                 // decode: key splits
+  int tcap;               // decode: cache rows
+};
+
+}  // namespace dla

@@ -1,0 +1,225 @@
+// Kernels on the fp32 residual stream of per-layer designs: scaled embedding, the stream update +
+// RMS norm, the per-layer token input's gate, squared ReLU.
+#include "mma.h"
+
+namespace dla {
+namespace {
+
+template <typename T>
+__global__ __launch_bounds__(256) void embed_stream_kernel(const int64_t* __restrict__ ids, const T* __restrict__ table,
+                                                           float scale, float* __restrict__ out, int* __restrict__ bad,
+                                                           int64_t V, int H) {
+  const int64_t row = blockIdx.x;
+  const int64_t id = ids[row];
+  const bool ok = id >= 0 && id < V;
+  if (!ok && threadIdx.x == 0) bad[0] = 1;
+  for (int c = threadIdx.x; c < H; c += blockDim.x)
+    out[row * H + c] = ok ? to_f<T>(table[id * H + c]) * scale : 0.f;
+}
+
+template <int NT>
+__device__ __forceinline__ float row_sum(float v, float* scratch) {
+  if constexpr (NT == 64) return wave_sum(v);
+  return block_sum<NT>(v, scratch);
+}
+
+// One row per workgroup, kept in registers (H % 4 == 0, H <= 4 * NT * NV).
+//   x += delta                       (DW: RMSNorm(delta) * delta_w)
+//   x += inject
+//   y = RMSNorm(x) * (offset + w)    (w == nullptr: y = x)
+template <typename T, int NT, int NV>
+__global__ __launch_bounds__(NT) void stream_norm_kernel(float* __restrict__ x, const T* __restrict__ delta,
+                                                         const T* __restrict__ delta_w, const float* __restrict__ inject,
+                                                         const T* __restrict__ w, T* __restrict__ y, float eps,
+                                                         float offset, int H) {
+  __shared__ float scratch[NT / 64];
+  const int64_t base = static_cast<int64_t>(blockIdx.x) * H;
+  float xv[NV][4], dv[NV][4];
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = 4 * (threadIdx.x + NT * j);
+    if (c < H) load_vec<float, 4>(x + base + c, xv[j]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) dv[j][e] = 0.f;
+    if (c < H && delta) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) dv[j][e] = to_f<T>(delta[base + c + e]);
+    }
+  }
+  if (delta_w) {
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss += dv[j][e] * dv[j][e];
+    const float r = rsqrtf(row_sum<NT>(ss, scratch) / H + eps);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int c = 4 * (threadIdx.x + NT * j);
+      if (c < H) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) dv[j][e] *= r * to_f<T>(delta_w[c + e]);
+      }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = 4 * (threadIdx.x + NT * j);
+    if (c >= H) continue;
+    float iv[4] = {0.f, 0.f, 0.f, 0.f};
+    if (inject) load_vec<float, 4>(inject + base + c, iv);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      xv[j][e] = xv[j][e] + dv[j][e] + iv[e];
+      ss += xv[j][e] * xv[j][e];
+    }
+    if (delta || inject) store_vec<float, 4>(x + base + c, xv[j]);
+  }
+  const float r = w ? rsqrtf(row_sum<NT>(ss, scratch) / H + eps) : 1.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = 4 * (threadIdx.x + NT * j);
+    if (c >= H) continue;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const float v = w ? xv[j][e] * r * (offset + to_f<T>(w[c + e])) : xv[j][e];
+      y[base + c + e] = from_f<T>(v);
+    }
+  }
+}
+
+// Any H: the row is read again from memory instead of kept (each thread re-reads its own elements).
+template <typename T>
+__global__ __launch_bounds__(256) void stream_norm_any_kernel(float* __restrict__ x, const T* __restrict__ delta,
+                                                              const T* __restrict__ delta_w,
+                                                              const float* __restrict__ inject, const T* __restrict__ w,
+                                                              T* __restrict__ y, float eps, float offset, int H) {
+  __shared__ float scratch[4];
+  const int64_t base = static_cast<int64_t>(blockIdx.x) * H;
+  float dr = 1.f;
+  if (delta_w) {
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < H; c += 256) {
+      const float d = to_f<T>(delta[base + c]);
+      ss += d * d;
+    }
+    dr = rsqrtf(block_sum<256>(ss, scratch) / H + eps);
+  }
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < H; c += 256) {
+    float v = x[base + c];
+    if (delta) v += delta_w ? to_f<T>(delta[base + c]) * (dr * to_f<T>(delta_w[c])) : to_f<T>(delta[base + c]);
+    if (inject) v += inject[base + c];
+    ss += v * v;
+    if (delta || inject) x[base + c] = v;
+  }
+  const float r = w ? rsqrtf(block_sum<256>(ss, scratch) / H + eps) : 1.f;
+  for (int c = threadIdx.x; c < H; c += 256) {
+    const float v = x[base + c];
+    y[base + c] = from_f<T>(w ? v * r * (offset + to_f<T>(w[c])) : v);
+  }
+}
+
+__device__ __forceinline__ float gelu_tanh(float z) {
+  return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void side_gate_kernel(const T* __restrict__ z, const int64_t* __restrict__ ids,
+                                                        const T* __restrict__ table, int64_t ldt, int64_t off,
+                                                        T* __restrict__ out, int64_t n, int dim, int64_t V) {
+  for (int64_t i = blockIdx.x * 256ll + threadIdx.x; i < n; i += gridDim.x * 256ll) {
+    const int64_t row = i / dim;
+    const int64_t id = ids[row];
+    const float e = id >= 0 && id < V ? to_f<T>(table[id * ldt + off + (i - row * dim)]) : 0.f;
+    out[i] = from_f<T>(gelu_tanh(to_f<T>(z[i])) * e);
+  }
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void relu2_kernel(const T* __restrict__ u, T* __restrict__ y, int64_t n) {
+  for (int64_t i = (blockIdx.x * 256ll + threadIdx.x) * VEC; i < n; i += gridDim.x * 256ll * VEC) {
+    float v[VEC];
+    load_vec<T, VEC>(u + i, v);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) {
+      const float r = fmaxf(v[e], 0.f);
+      v[e] = r * r;
+    }
+    store_vec<T, VEC>(y + i, v);
+  }
+}
+
+inline unsigned grid_for(int64_t work) {
+  const int64_t b = (work + 255) / 256;
+  return static_cast<unsigned>(b < 1 ? 1 : (b > 8192 ? 8192 : b));
+}
+
+template <typename T>
+void norm_dispatch(float* x, const T* delta, const T* dw, const float* inject, const T* w, T* y, float eps,
+                   float offset, int64_t rows, int H, hipStream_t st) {
+  const dim3 g(static_cast<unsigned>(rows));
+#define DLA_NORM(NT, NV) stream_norm_kernel<T, NT, NV><<<g, NT, 0, st>>>(x, delta, dw, inject, w, y, eps, offset, H)
+  if (H % 4 || H > 16384) stream_norm_any_kernel<T><<<g, 256, 0, st>>>(x, delta, dw, inject, w, y, eps, offset, H);
+  else if (H <= 256) DLA_NORM(64, 1);
+  else if (H <= 1024) DLA_NORM(256, 1);
+  else if (H <= 2048) DLA_NORM(256, 2);
+  else if (H <= 4096) DLA_NORM(256, 4);
+  else if (H <= 8192) DLA_NORM(256, 8);
+  else DLA_NORM(1024, 4);
+#undef DLA_NORM
+}
+
+}  // namespace
+
+void launch_embed_stream(bool bf16, const int64_t* ids, const void* table, float scale, float* out, int* bad,
+                         int64_t rows, int64_t V, int H, hipStream_t st) {
+  if (rows == 0) return;
+  const dim3 g(static_cast<unsigned>(rows));
+  if (bf16) embed_stream_kernel<bf16_t><<<g, 256, 0, st>>>(ids, static_cast<const bf16_t*>(table), scale, out, bad, V, H);
+  else embed_stream_kernel<float><<<g, 256, 0, st>>>(ids, static_cast<const float*>(table), scale, out, bad, V, H);
+}
+
+void launch_stream_norm(bool bf16, float* x, const void* delta, const void* dw, const float* inject, const void* w,
+                        void* y, float eps, float offset, int64_t rows, int H, hipStream_t st) {
+  if (rows == 0) return;
+  if (bf16)
+    norm_dispatch<bf16_t>(x, static_cast<const bf16_t*>(delta), static_cast<const bf16_t*>(dw), inject,
+                          static_cast<const bf16_t*>(w), static_cast<bf16_t*>(y), eps, offset, rows, H, st);
+  else
+    norm_dispatch<float>(x, static_cast<const float*>(delta), static_cast<const float*>(dw), inject,
+                         static_cast<const float*>(w), static_cast<float*>(y), eps, offset, rows, H, st);
+}
+
+void launch_side_gate(bool bf16, const void* z, const int64_t* ids, const void* table, int64_t ldt, int64_t off,
+                      void* out, int64_t rows, int dim, int64_t V, hipStream_t st) {
+  const int64_t n = rows * dim;
+  if (n == 0) return;
+  if (bf16)
+    side_gate_kernel<bf16_t><<<grid_for(n), 256, 0, st>>>(static_cast<const bf16_t*>(z), ids,
+                                                          static_cast<const bf16_t*>(table), ldt, off,
+                                                          static_cast<bf16_t*>(out), n, dim, V);
+  else
+    side_gate_kernel<float><<<grid_for(n), 256, 0, st>>>(static_cast<const float*>(z), ids,
+                                                         static_cast<const float*>(table), ldt, off,
+                                                         static_cast<float*>(out), n, dim, V);
+}
+
+void launch_relu2(bool bf16, const void* u, void* y, int64_t n, hipStream_t st) {
+  if (n == 0) return;
+  const bool vec = n % 8 == 0 && reinterpret_cast<uintptr_t>(u) % 16 == 0 && reinterpret_cast<uintptr_t>(y) % 16 == 0;
+  if (bf16) {
+    const bf16_t* up = static_cast<const bf16_t*>(u);
+    bf16_t* yp = static_cast<bf16_t*>(y);
+    if (vec) relu2_kernel<bf16_t, 8><<<grid_for(n / 8), 256, 0, st>>>(up, yp, n);
+    else relu2_kernel<bf16_t, 1><<<grid_for(n), 256, 0, st>>>(up, yp, n);
+  } else {
+    const float* up = static_cast<const float*>(u);
+    float* yp = static_cast<float*>(y);
+    if (vec) relu2_kernel<float, 8><<<grid_for(n / 8), 256, 0, st>>>(up, yp, n);
+    else relu2_kernel<float, 1><<<grid_for(n), 256, 0, st>>>(up, yp, n);
+  }
+}
+
+}  // namespace dla

@@ -11,12 +11,12 @@ import dataclasses
 import json
 from dataclasses import dataclass, field
 from pathlib import Path
-from typing import Any, Dict, Optional
+from typing import Any, Dict, List, Optional, Tuple
 
 
 @dataclass
 class ModelConfig:
-    arch: str = "llama"  # llama | mistral | mixtral | gpt2 | phi
+    arch: str = "llama"  # llama | mistral | mixtral | gpt2 | phi | vufilorn
     vocab_size: int = 32000
     hidden_size: int = 4096
     num_layers: int = 32
@@ -35,7 +35,7 @@ class ModelConfig:
     num_experts_per_tok: int = 2
     router_aux_loss_coef: float = 0.0
     norm_type: str = "rms"  # rms | layer
-    activation: str = "swiglu"  # swiglu | gelu_new
+    activation: str = "swiglu"  # swiglu | gelu_new | relu2
     parallel_block: bool = False  # phi: attn and mlp both read the same normed input
     attn_bias: bool = False
     mlp_bias: bool = False
@@ -46,6 +46,28 @@ class ModelConfig:
     pad_token_id: Optional[int] = None
     init_std: float = 0.02
     name: str = "custom"
+    # per-layer designs (models/mixers.py): one {"type", "mixer", "mlp"} dict per layer, each with
+    # its own sizes; None = num_layers equal DecoderLayers described by the fields above
+    layer_specs: Optional[List[Dict[str, Any]]] = None
+    loop: Optional[Dict[str, int]] = None  # layers start .. stop-1 run `times` times in a row
+    embed_scale: float = 1.0
+    norm_offset: float = 0.0  # added to the stored norm weights (1.0: weights stored around zero)
+    token_side_dim: int = 0  # per-layer token input: width of each layer's slice of side_embed
+
+    @property
+    def layer_schedule(self) -> List[Tuple[int, bool]]:
+        """The layer runs of one forward in order: (layer index, whether the embedding output is
+        added to the stream first). Every run has its own cache / state slot."""
+        n = self.num_layers
+        if not self.loop:
+            return [(i, False) for i in range(n)]
+        a, b, times = int(self.loop["start"]), int(self.loop["stop"]), int(self.loop["times"])
+        if not (0 <= a < b <= n and times >= 1):
+            raise ValueError(f"loop {self.loop} does not fit {n} layers")
+        runs = [(i, False) for i in range(a)]
+        for p in range(times):
+            runs += [(i, p > 0 and i == a) for i in range(a, b)]
+        return runs + [(i, False) for i in range(b, n)]
 
     @property
     def q_size(self) -> int:
@@ -66,6 +88,12 @@ class ModelConfig:
         return self.num_experts > 0
 
     def num_params(self, include_embedding: bool = True) -> int:
+        if self.layer_specs is not None:
+            from .layer_spec import spec_param_count
+
+            H, L, V = self.hidden_size, self.num_layers, self.vocab_size
+            n = H + sum(spec_param_count(self, i) for i in range(L))
+            return n + (V * H + V * L * self.token_side_dim if include_embedding else 0)
         H, F, L = self.hidden_size, self.intermediate_size, self.num_layers
         attn = H * (self.q_size + 2 * self.kv_size) + self.q_size * H
         mlp_one = (3 if self.activation == "swiglu" else 2) * H * F
@@ -78,6 +106,11 @@ class ModelConfig:
 
     def flops_per_token(self, seq_len: int) -> float:
         """Forward FLOPs/token: 2*matmul params (active experts only) + causal attention."""
+        if self.layer_specs is not None:
+            from .layer_spec import spec_flops_per_token
+
+            return (2.0 * self.vocab_size * self.hidden_size
+                    + sum(spec_flops_per_token(self, i, seq_len) for i, _ in self.layer_schedule))
         H, F, L = self.hidden_size, self.intermediate_size, self.num_layers
         attn_proj = H * (self.q_size + 2 * self.kv_size) + self.q_size * H
         n_mlp = self.num_experts_per_tok if self.is_moe else 1
@@ -97,6 +130,8 @@ class ModelConfig:
     # ----------------------------------------------------------------- HF config.json interop
     @classmethod
     def from_hf(cls, hf: Dict[str, Any]) -> "ModelConfig":
+        if hf.get("architecture") == "Vufilorn":
+            return cls._from_vufilorn(hf)
         mt = hf.get("model_type", "llama")
         if mt in ("llama", "mistral", "mixtral", "qwen2"):
             H = hf["hidden_size"]
@@ -146,7 +181,42 @@ class ModelConfig:
             )
         raise ValueError(f"unsupported model_type {mt!r}")
 
+    @classmethod
+    def _from_vufilorn(cls, d: Dict[str, Any]) -> "ModelConfig":
+        """Vufilorn config.json: `layers` lists each layer's mixer (latent attention or retention)
+        and feed-forward with their own sizes; the flat head / FFN fields get the largest of them
+        (reporting only, the layers read their specs)."""
+        from .layer_spec import check_spec
+
+        specs = [dict(e) for e in d["layers"]]
+        for i, e in enumerate(specs):
+            check_spec(e, i)
+        mix = [e["mixer"] for e in specs]
+        return cls(
+            arch="vufilorn", vocab_size=d["vocab"], hidden_size=d["width"], num_layers=len(specs),
+            num_heads=max(m["heads"] for m in mix), num_kv_heads=max(m["heads"] for m in mix),
+            head_dim=max(m["dim"] + m.get("rot_dim", 0) for m in mix),
+            intermediate_size=max([e["mlp"]["ff"] for e in specs if e.get("mlp")], default=0),
+            norm_eps=d["norm"]["eps"], norm_offset=1.0, activation="relu2", tie_word_embeddings=True,
+            max_position_embeddings=d.get("max_position_embeddings", 131072),
+            layer_specs=specs, loop=d.get("loop"), embed_scale=float((d.get("embedding") or {}).get("scale", 1.0)),
+            token_side_dim=int((d.get("token_side") or {}).get("dim", 0)),
+            # the design names no special tokens: -1 = never sampled, generation runs to its length
+            bos_token_id=d.get("bos_token_id", -1), eos_token_id=d.get("eos_token_id", -1), name="vufilorn")
+
+    def _to_vufilorn(self) -> Dict[str, Any]:
+        d = {"architecture": "Vufilorn", "vocab": self.vocab_size, "width": self.hidden_size,
+             "embedding": {"scale": self.embed_scale}, "norm": {"eps": self.norm_eps},
+             "layers": [dict(e) for e in self.layer_specs], "loop": self.loop,
+             "token_side": {"dim": self.token_side_dim} if self.token_side_dim else None}
+        for k in ("bos_token_id", "eos_token_id"):
+            if getattr(self, k) >= 0:
+                d[k] = getattr(self, k)
+        return d
+
     def to_hf(self) -> Dict[str, Any]:
+        if self.arch == "vufilorn":
+            return self._to_vufilorn()
         if self.arch == "gpt2":
             return {"model_type": "gpt2", "architectures": ["GPT2LMHeadModel"], "vocab_size": self.vocab_size,
                     "n_embd": self.hidden_size, "n_layer": self.num_layers, "n_head": self.num_heads,
@@ -186,6 +256,21 @@ class ModelConfig:
 
 def _first(x):
     return x[0] if isinstance(x, (list, tuple)) else x
+
+
+def _vufilorn_preset(vocab, width, order, ff, latent, retention, side_dim, scale, loop=None, eps=1e-6):
+    """PRESETS entry of a Vufilorn model: `order` is one letter per layer, L(atent attention) or
+    R(etention), all layers of a kind with the same sizes."""
+    lat = {"type": "latent_attention", "mixer": latent, "mlp": {"kind": "dense", "ff": ff}}
+    ret = {"type": "retention", "mixer": retention, "mlp": {"kind": "dense", "ff": ff}}
+    return ModelConfig._from_vufilorn({
+        "vocab": vocab, "width": width, "embedding": {"scale": scale}, "norm": {"eps": eps}, "loop": loop,
+        "token_side": {"dim": side_dim}, "layers": [lat if c == "L" else ret for c in order]}).to_dict()
+
+
+def _decays(heads: int, lo: float = 1 / 32, hi: float = 1 / 512) -> List[float]:
+    """`heads` decays 1 - x, x log-spaced from lo to hi."""
+    return [1.0 - lo * (hi / lo) ** (h / max(1, heads - 1)) for h in range(heads)]
 
 
 PRESETS: Dict[str, Dict[str, Any]] = {
@@ -241,6 +326,28 @@ PRESETS: Dict[str, Dict[str, Any]] = {
                      bos_token_id=1, eos_token_id=2),
 }
 
+PRESETS.update({
+    # Vufilorn (latent attention in a window + retention, looped layers, per-layer token input)
+    "tiny-vufilorn": _vufilorn_preset(
+        320, 96, "RLL", 160,
+        dict(heads=3, dim=16, rot_dim=8, vdim=24, kv_rank=40, q_rank=32, scale=0.2,
+             rot=dict(base=10000.0, dims=8), mask=dict(size=11)),
+        dict(heads=2, dim=24, vdim=40, rot=dict(base=500.0, dims=16), decay=[0.9, 0.97]),
+        side_dim=8, scale=3.0, loop=dict(start=1, stop=3, times=2)),
+    "vufilorn-1b": _vufilorn_preset(
+        32000, 2048, "LRLRLRLRLRLR", 8192,
+        dict(heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=768, scale=192 ** -0.5,
+             rot=dict(base=1e6, dims=64), mask=dict(size=4096)),
+        dict(heads=16, dim=128, vdim=128, rot=dict(base=1e6, dims=128), decay=_decays(16)),
+        side_dim=128, scale=45.0, loop=dict(start=2, stop=10, times=2)),
+    "vufilorn-7b": _vufilorn_preset(
+        32000, 4096, "LRLRLRLRLRLRLRLRLRLR", 16384,
+        dict(heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1536, scale=192 ** -0.5,
+             rot=dict(base=1e6, dims=64), mask=dict(size=4096)),
+        dict(heads=16, dim=256, vdim=256, rot=dict(base=1e6, dims=256), decay=_decays(16)),
+        side_dim=256, scale=64.0, loop=dict(start=4, stop=16, times=2)),
+})
+
 # HF hub ids used by the reference configs -> presets (random init offline, identical shapes)
 HUB_ALIASES = {
     "mistralai/Mistral-7B-v0.1": "mistral-7b",
@@ -259,6 +366,8 @@ def tp_shard_config(cfg: ModelConfig, tp: int) -> ModelConfig:
     (world-1) model: heads, KV heads, FFN width and vocabulary divided by tp, hidden size and
     depth kept. Used by `bench.py --tp-shape` to time one TP rank's real GEMM / attention / norm
     shapes on one GPU (e.g. Llama-3-70B at tp 8: 8 q heads / 1 kv head, FFN 3584, vocab 16032)."""
+    if cfg.layer_specs is not None:
+        raise ValueError(f"{cfg.name}: per-layer designs have no tensor-parallel form")
     if cfg.num_heads % tp or cfg.num_kv_heads % tp or cfg.intermediate_size % tp or cfg.vocab_size % tp:
         raise ValueError(f"{cfg.name}: heads / kv heads / FFN / vocab must divide tp={tp}")
     d = cfg.to_dict()
@@ -290,7 +399,7 @@ def get_config(name_or_path: str, **overrides) -> ModelConfig:
         key = HUB_ALIASES.get(str(name_or_path), str(name_or_path))
         if key not in PRESETS:
             raise KeyError(f"unknown model {name_or_path!r}; presets: {sorted(PRESETS)}")
-        cfg = ModelConfig(**PRESETS[key], name=key)
+        cfg = ModelConfig(**{**PRESETS[key], "name": key})
     for k, v in overrides.items():
         setattr(cfg, k, v)
     return cfg

@@ -23,7 +23,10 @@ from .transformer import CausalLM, attention_layout
 
 
 class KVCache:
-    """Contiguous per-layer K/V cache [L, B, T_max, Hkv, D] sized once for prompt + new tokens.
+    """What a batch of left-padded sequences keeps of its past.
+
+    Attention families: contiguous per-layer K/V cache [L, B, T_max, Hkv, D] sized once for prompt + new tokens.
+    Per-layer designs: `slots`, one per layer run, made by the layer's mixer (models/mixers.py).
 
     The write slot, attended length and next positions also live on the device (`slot`,
     `kv_len`, `pos`), so a single-token decode step touches no host value: it can be captured
@@ -32,10 +35,30 @@ class KVCache:
     def __init__(self, model: CausalLM, batch: int, max_len: int, kv_start: Optional[torch.Tensor]):
         cfg = model.cfg
         dev, dt = model.embed.device, model.embed.dtype
-        L, Hkv, D = cfg.num_layers, model.layers[0].attn.kv_local, cfg.head_dim
-        self.h_local, self.kv_local = model.layers[0].attn.h_local, Hkv
         self.cfg = cfg
         self.split = model.layer_devices is not None
+        self.k = self.v = self.slots = None
+        if cfg.layer_specs is not None:
+            # per-layer designs: one slot per layer run (latents of every token, or fixed-size state)
+            self.slots = [model.layers[i].mix.new_slot(batch, max_len, dev, dt) for i, _ in model.schedule]
+            fast = dev.type == "cuda"
+        else:
+            fast = self._alloc_kv(model, batch, max_len, dev, dt)
+        self.max_len = max_len
+        self.len = 0
+        self.batch = batch
+        self.kv_start = kv_start.to(torch.int32).clone() if kv_start is not None else None
+        self._pos = None
+        self.slot = torch.zeros(1, dtype=torch.long, device=dev)
+        self.kv_len = torch.ones(1, dtype=torch.int32, device=dev)
+        self.pos = torch.zeros((batch, 1), dtype=torch.int32, device=dev)
+        self.fast_decode = fast
+
+    def _alloc_kv(self, model, batch: int, max_len: int, dev, dt) -> bool:
+        """Per-layer K/V of the attention families; returns whether the decode kernels take them."""
+        cfg = self.cfg
+        L, Hkv, D = cfg.num_layers, model.layers[0].attn.kv_local, cfg.head_dim
+        self.h_local, self.kv_local = model.layers[0].attn.h_local, Hkv
         if self.split:  # layer-split model: each layer's K/V on that layer's device
             self.k = [torch.empty((batch, max_len, Hkv, D), device=d, dtype=dt) for d in model.layer_devices]
             self.v = [torch.empty((batch, max_len, Hkv, D), device=d, dtype=dt) for d in model.layer_devices]
@@ -48,18 +71,12 @@ class KVCache:
         else:
             self.k = torch.empty((L, batch, max_len, Hkv, D), device=dev, dtype=dt)
             self.v = torch.empty((L, batch, max_len, Hkv, D), device=dev, dtype=dt)
-        self.max_len = max_len
-        self.len = 0
-        self.batch = batch
-        self.kv_start = kv_start.to(torch.int32).clone() if kv_start is not None else None
-        self._pos = None
-        self.slot = torch.zeros(1, dtype=torch.long, device=dev)
-        self.kv_len = torch.ones(1, dtype=torch.int32, device=dev)
-        self.pos = torch.zeros((batch, 1), dtype=torch.int32, device=dev)
-        self.fast_decode = (not self.split and dev.type == "cuda" and dt == torch.bfloat16
-                            and ops.decode.decode_supported(self.h_local, Hkv, D))
+        return (not self.split and dev.type == "cuda" and dt == torch.bfloat16
+                and ops.decode.decode_supported(self.h_local, Hkv, D))
 
     def nbytes(self) -> int:
+        if self.slots is not None:
+            return sum(s.nbytes() for s in self.slots)
         ks = self.k if isinstance(self.k, list) else [self.k]
         return 2 * sum(t.numel() * t.element_size() for t in ks)
 
@@ -71,6 +88,32 @@ class KVCache:
         self.capturing = False
         if kv_start is not None:
             self.kv_start.copy_(kv_start.to(torch.int32))
+
+    def reserve(self, max_len: int):
+        """Make room for max_len tokens per row (slot caches; grown geometrically). Not while a
+        captured decode step reads this cache."""
+        if self.slots is None or max_len <= self.max_len:
+            return
+        if self.capturing:
+            raise RuntimeError("KV cache overflow")
+        self.max_len = max(max_len, self.max_len + self.max_len // 2)
+        for s in self.slots:
+            s.reserve(self.max_len)
+
+    def keep_rows(self, rows) -> "KVCache":
+        """A cache of the given batch rows only (slot caches): what the other rows hold is given back
+        once this one is dropped."""
+        if self.slots is None:
+            raise NotImplementedError("keep_rows: slot caches only")
+        rows = torch.as_tensor(rows, dtype=torch.long, device=self.slot.device)
+        out = KVCache.__new__(KVCache)
+        out.__dict__.update(self.__dict__)
+        out.slots = [s.keep_rows(rows) for s in self.slots]
+        out.batch = int(rows.numel())
+        out.kv_start = self.kv_start.index_select(0, rows) if self.kv_start is not None else None
+        out.pos = self.pos.index_select(0, rows)
+        out.slot, out.kv_len, out._pos = self.slot.clone(), self.kv_len.clone(), None
+        return out
 
     def positions_for(self, T: int) -> torch.Tensor:
         if T == 1 and self.len > 0:
@@ -191,7 +234,7 @@ def _graph_capable(model: CausalLM) -> bool:
 
 def _graph_ok(model: CausalLM, cache: KVCache) -> bool:
     return (cache.fast_decode and _graph_capable(model) and not cache.split
-            and ops._ext.use_native(cache.k))
+            and ops._ext.use_native(cache.slot))
 
 
 class _DecodeGraph:
@@ -199,7 +242,7 @@ class _DecodeGraph:
     -> norm -> LM head -> fused sampler -> finished/pad bookkeeping, all on device."""
 
     def __init__(self, model, cache, B, max_new, eos, pad, greedy, temperature, top_k, top_p, seed):
-        dev = cache.k.device
+        dev = cache.slot.device
         self.model, self.cache = model, cache
         self.tok = torch.zeros((B, 1), dtype=torch.long, device=dev)
         self.finished = torch.zeros(B, dtype=torch.bool, device=dev)

@@ -80,6 +80,29 @@ def _layer_map(cfg, i: int) -> List[Tuple[str, str, tuple]]:
             (n + "mlp.down_proj", p + "mlp.c_proj.weight", "T"),
             (n + "mlp.down_bias", p + "mlp.c_proj.bias", None),
         ]
+    if cfg.arch == "vufilorn":
+        spec, p = cfg.layer_specs[i], f"l{i}."
+        x = spec["mixer"]
+        m = [(n + "ln1_w", p + "norm1", None)]
+        if spec["type"] == "latent_attention":
+            a, b = x["q_rank"], x["q_rank"] + x["kv_rank"] + x["rot_dim"]
+            k, v = x["heads"] * x["dim"], x["heads"] * (x["dim"] + x["vdim"])
+            m += [(n + "mix.in_proj", p + "mix.dq", (0, a)), (n + "mix.in_proj", p + "mix.dkv", (a, b)),
+                  (n + "mix.q_norm_w", p + "mix.dq.norm", None), (n + "mix.kv_norm_w", p + "mix.dkv.norm", None),
+                  (n + "mix.q_up", p + "mix.uq", None),
+                  (n + "mix.kv_up", p + "mix.uk", (0, k)), (n + "mix.kv_up", p + "mix.uv", (k, v))]
+        else:
+            k, v = x["heads"] * x["dim"], x["heads"] * x["vdim"]
+            m += [(n + "mix.qkvg_proj", p + "mix." + t, (a, b)) for t, a, b in
+                  (("q", 0, k), ("k", k, 2 * k), ("v", 2 * k, 2 * k + v), ("g", 2 * k + v, 2 * (k + v)))]
+        m.append((n + "mix.o_proj", p + "mix.o", None))
+        if spec.get("mlp"):
+            m += [(n + "ln2_w", p + "norm2", None), (n + "mlp.up_proj", p + "mlp.up", None),
+                  (n + "mlp.down_proj", p + "mlp.down", None)]
+        if cfg.token_side_dim:
+            m += [(n + "side.gate", p + "side.gate", None), (n + "side.proj", p + "side.proj", None),
+                  (n + "side.norm_w", p + "side.norm", None)]
+        return m
     raise ValueError(cfg.arch)
 
 
@@ -92,6 +115,10 @@ def _global_map(cfg) -> List[Tuple[str, str, tuple]]:
              ("norm_w", "model.final_layernorm.weight", None),
              ("norm_b", "model.final_layernorm.bias", None),
              ("lm_head", "lm_head.weight", None), ("lm_head_bias", "lm_head.bias", None)]
+    elif cfg.arch == "vufilorn":
+        m = [("embed", "embed", None), ("norm_w", "final.norm", None)]
+        if cfg.token_side_dim:
+            m.append(("side_embed", "side.embed", None))
     else:
         m = [("embed", "model.embed_tokens.weight", None), ("norm_w", "model.norm.weight", None)]
         if not cfg.tie_word_embeddings:

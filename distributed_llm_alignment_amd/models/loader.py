@@ -96,7 +96,7 @@ def load_causal_lm(model_name_or_path: str, gradient_checkpointing: bool = True,
         model = build_model(cfg, device=device, dtype=dtype, seed=seed, init=not has_weights, headless=headless)
         if has_weights:
             sd = read_state_dict(p)
-            model.load_hf_state_dict(sd, strict=False)
+            model.load_hf_state_dict(sd, strict=cfg.layer_specs is not None)
     if split is not None:
         dispatch_layers(model, split)
     if gradient_checkpointing:  # True / "full", or a selective policy ("mlp", "attention")

@@ -1,0 +1,233 @@
+"""Layers of per-layer designs (`ModelConfig.layer_specs`): latent attention and retention mixers,
+squared-ReLU / other feed-forwards, the per-layer token input, and the layer that strings them
+together on an fp32 residual stream.
+
+A `StreamLayer` never adds its own output to the stream: it hands the last projection's output on as
+the *pending* update of a `Stream`, and the next norm kernel adds it while it reads the stream (one
+pass: add, optional norm of the update, optional embedding re-injection, norm of the sum). Mixers
+keep what they need of the past in a slot of `generation.KVCache` (`new_slot`); a layer that runs
+several times per forward gets one slot per run.
+"""
+from __future__ import annotations
+
+import dataclasses
+import math
+from typing import List, Optional
+
+import torch
+import torch.nn as nn
+
+from .. import ops
+from .config import ModelConfig
+from .layer_spec import window
+
+
+def _param(*shape, device=None, dtype=None) -> nn.Parameter:
+    return nn.Parameter(torch.empty(*shape, device=device, dtype=dtype))
+
+
+@dataclasses.dataclass
+class Stream:
+    """fp32 residual stream x [B, T, H] plus the update not added yet: x + norm?(delta) + inject."""
+
+    x: torch.Tensor
+    delta: Optional[torch.Tensor] = None
+    delta_w: Optional[torch.Tensor] = None  # plain RMS norm of delta with this weight before the add
+    inject: Optional[torch.Tensor] = None
+    ssq: Optional[torch.Tensor] = None      # decode: partial sums of squares of x's rows
+
+    def norm(self, w, eps: float, offset: float, dtype) -> torch.Tensor:
+        """Fold the pending update into x and return the normed rows."""
+        y, self.x = ops.stream_norm(self.x, self.delta, self.delta_w, self.inject, w, eps, offset, dtype)
+        self.delta = self.delta_w = self.inject = self.ssq = None
+        return y
+
+    def cast(self, eps: float, dtype) -> torch.Tensor:
+        """Fold the pending update into x and return x in the compute dtype."""
+        return self.norm(None, eps, 0.0, dtype)
+
+
+class CacheSlot:
+    """What one mixer run keeps of the past: named tensors with the batch first. `time_dim` tensors
+    have one row per token (grown by `reserve`), the others are fixed-size state."""
+
+    def __init__(self, rope, max_len: int, device, **tensors):
+        self.t = tensors
+        self.rope = rope
+        self.grow(max_len, device)
+
+    def grow(self, max_len: int, device):
+        # the slot keeps its own reference to the rotary tables: a captured decode step reads them
+        # by address, also after a longer cache made the shared RotaryCache extend
+        self.rope.ensure(max_len)
+        self.cos, self.sin = self.rope.tables(device)
+
+    def nbytes(self) -> int:
+        return sum(v.numel() * v.element_size() for v in self.t.values())
+
+    def keep_rows(self, rows: torch.Tensor) -> "CacheSlot":
+        out = CacheSlot.__new__(CacheSlot)
+        out.rope, out.cos, out.sin = self.rope, self.cos, self.sin
+        out.t = {k: v.index_select(0, rows.to(v.device)) for k, v in self.t.items()}
+        return out
+
+    def reserve(self, max_len: int):
+        if "latent" in self.t:
+            old = self.t["latent"]
+            new = torch.zeros((old.shape[0], max_len, old.shape[2]), dtype=old.dtype, device=old.device)
+            new[:, :old.shape[1]] = old
+            self.t["latent"] = new
+            self.grow(max_len, old.device)
+        else:
+            self.grow(max_len, self.t["state"].device)
+
+
+class LatentAttention(nn.Module):
+    """Multi-head attention whose keys and values are projections of one cached latent per token
+    (plus one rotated key part shared by the heads), inside a sliding window."""
+
+    def __init__(self, cfg: ModelConfig, m: dict, device=None, dtype=None):
+        super().__init__()
+        H = cfg.hidden_size
+        self.eps = cfg.norm_eps
+        self.heads, self.dim, self.rot, self.vdim = m["heads"], m["dim"], m["rot_dim"], m["vdim"]
+        self.q_rank, self.kv_rank = m["q_rank"], m["kv_rank"]
+        self.scale, self.window = float(m["scale"]), window(m)
+        self.rope_key = (m["rot"]["dims"], float(m["rot"]["base"]))
+        self.rope = None  # the model's shared RotaryCache of rope_key
+        self.in_proj = _param(self.q_rank + self.kv_rank + self.rot, H, device=device, dtype=dtype)
+        self.q_norm_w = _param(self.q_rank, device=device, dtype=dtype)
+        self.kv_norm_w = _param(self.kv_rank, device=device, dtype=dtype)
+        self.q_up = _param(self.heads * (self.dim + self.rot), self.q_rank, device=device, dtype=dtype)
+        # [all heads' unrotated keys; all heads' values]
+        self.kv_up = _param(self.heads * (self.dim + self.vdim), self.kv_rank, device=device, dtype=dtype)
+        self.o_proj = _param(H, self.heads * self.vdim, device=device, dtype=dtype)
+
+    def new_slot(self, batch: int, max_len: int, device, dtype) -> CacheSlot:
+        return CacheSlot(self.rope, max_len, device, latent=torch.zeros(
+            (batch, max_len, self.kv_rank + self.rot), device=device, dtype=dtype))
+
+    def attend(self, down: torch.Tensor, cache, slot: CacheSlot) -> torch.Tensor:
+        """down = in_proj output [B, T, q_rank + kv_rank + rot] -> heads' outputs [B, T, heads * vdim];
+        the new tokens' latents go into the slot."""
+        B, T, _ = down.shape
+        latent = slot.t["latent"]
+        cq = ops.latent.prepare(down, self.q_norm_w, self.kv_norm_w, self.eps, latent, cache.slot,
+                                cache.kv_start, slot.cos, slot.sin, base=cache.len)
+        q = ops.stream_linear(cq, self.q_up)
+        if T == 1 and cache.len > 0:
+            return ops.latent.decode(q, latent, self.kv_up, self.heads, self.dim, self.rot, self.vdim,
+                                     self.scale, self.window, cache.slot, cache.kv_start, slot.cos,
+                                     slot.sin, base=cache.len)
+        # prefill (of a whole prompt, or a portion after earlier ones): keys and values of every
+        # visible token are projected up once
+        lo = max(0, cache.len + 1 - self.window) if self.window else 0
+        seen = latent[:, lo:cache.len + T]
+        kv = ops.stream_linear(seen[..., :self.kv_rank].contiguous(), self.kv_up)
+        return ops.latent.prefill(q, kv, seen[..., self.kv_rank:], self.heads, self.dim, self.rot, self.vdim,
+                                  self.scale, self.window, cache.kv_start, slot.cos, slot.sin,
+                                  q_base=cache.len, k_base=lo)
+
+    def forward(self, h, cache, slot):
+        a = self.attend(ops.stream_linear(h, self.in_proj), cache, slot)
+        return ops.stream_linear(a, self.o_proj)
+
+
+class Retention(nn.Module):
+    """Linear attention with one fixed decay per head; its past is one fp32 state per head."""
+
+    def __init__(self, cfg: ModelConfig, m: dict, device=None, dtype=None):
+        super().__init__()
+        H = cfg.hidden_size
+        self.eps = cfg.norm_eps
+        self.heads, self.dim, self.vdim = m["heads"], m["dim"], m["vdim"]
+        self.rope_key = (m["rot"]["dims"], float(m["rot"]["base"]))
+        self.rope = None
+        self.decay = [float(x) for x in m["decay"]]
+        self._decay = {}
+        # rows [q; k; v; g]
+        self.qkvg_proj = _param(2 * self.heads * (self.dim + self.vdim), H, device=device, dtype=dtype)
+        self.o_proj = _param(H, self.heads * self.vdim, device=device, dtype=dtype)
+
+    def decays(self, device) -> torch.Tensor:
+        """[2, heads] fp32: the decays and their base-2 logarithms."""
+        t = self._decay.get(device)
+        if t is None:
+            d = torch.tensor(self.decay, dtype=torch.float64)
+            t = torch.stack([d, d.log2().clamp(min=-1e4)]).float().to(device)
+            self._decay[device] = t
+        return t
+
+    def new_slot(self, batch: int, max_len: int, device, dtype) -> CacheSlot:
+        return CacheSlot(self.rope, max_len, device, state=torch.zeros(
+            (batch, self.heads, self.vdim, self.dim), device=device, dtype=torch.float32))
+
+    def mix(self, qkvg: torch.Tensor, cache, slot: CacheSlot) -> torch.Tensor:
+        B, T, _ = qkvg.shape
+        args = (self.heads, self.dim, self.vdim, self.rope_key[0], self.eps, self.decays(qkvg.device),
+                slot.t["state"], cache.slot, cache.kv_start, slot.cos, slot.sin)
+        if T == 1 and cache.len > 0:
+            return ops.retention.decode(qkvg, *args, base=cache.len)
+        return ops.retention.prefill(qkvg, *args, base=cache.len)
+
+    def forward(self, h, cache, slot):
+        return ops.stream_linear(self.mix(ops.stream_linear(h, self.qkvg_proj), cache, slot), self.o_proj)
+
+
+MIXERS = {"latent_attention": LatentAttention, "retention": Retention}
+
+
+class TokenSide(nn.Module):
+    """Per-layer token input: a gated slice of a second embedding, projected up and RMS-normed."""
+
+    def __init__(self, cfg: ModelConfig, device=None, dtype=None):
+        super().__init__()
+        self.gate = _param(cfg.token_side_dim, cfg.hidden_size, device=device, dtype=dtype)
+        self.proj = _param(cfg.hidden_size, cfg.token_side_dim, device=device, dtype=dtype)
+        self.norm_w = _param(cfg.hidden_size, device=device, dtype=dtype)
+
+
+class StreamLayer(nn.Module):
+    """One layer of a per-layer design: norm, mixer, [norm, feed-forward], [per-layer token input]."""
+
+    def __init__(self, cfg: ModelConfig, index: int, device=None, dtype=None):
+        super().__init__()
+        from .transformer import MLP
+
+        spec = cfg.layer_specs[index]
+        self.cfg, self.index = cfg, index
+        H = cfg.hidden_size
+        self.ln1_w = _param(H, device=device, dtype=dtype)
+        self.mix = MIXERS[spec["type"]](cfg, spec["mixer"], device, dtype)
+        self.mlp = None
+        if spec.get("mlp"):
+            self.ln2_w = _param(H, device=device, dtype=dtype)
+            self.mlp = MLP(dataclasses.replace(cfg, intermediate_size=spec["mlp"]["ff"]), device, dtype)
+        self.side = TokenSide(cfg, device, dtype) if cfg.token_side_dim else None
+        self.recompute = None
+
+    def forward(self, s: Stream, ids: torch.Tensor, side_embed, cache, slot: CacheSlot) -> Stream:
+        cfg, dt = self.cfg, self.ln1_w.dtype
+        h = s.norm(self.ln1_w, cfg.norm_eps, cfg.norm_offset, dt)
+        s.delta = self.mix(h, cache, slot)
+        if self.mlp is not None:
+            h = s.norm(self.ln2_w, cfg.norm_eps, cfg.norm_offset, dt)
+            s.delta = self.mlp(h)
+        if self.side is not None:
+            side = self.side
+            g = ops.side_gate(ops.stream_linear(s.cast(cfg.norm_eps, dt), side.gate), ids, side_embed,
+                              self.index * cfg.token_side_dim)
+            s.delta, s.delta_w = ops.stream_linear(g, side.proj), side.norm_w
+        return s
+
+
+def build_layers(cfg: ModelConfig, device=None, dtype=None) -> List[StreamLayer]:
+    """The layers of a per-layer design; mixers with equal rotary settings share one table."""
+    layers = [StreamLayer(cfg, i, device, dtype) for i in range(cfg.num_layers)]
+    ropes = {}
+    for layer in layers:
+        key = layer.mix.rope_key
+        if key not in ropes:
+            ropes[key] = ops.RotaryCache(key[0], key[1], 256)
+        layer.mix.rope = ropes[key]
+    return layers

@@ -144,7 +144,7 @@ def load_tokenizer(name_or_path: str, cfg=None):
             tok.pad_token = tok.eos_token
         return tok
     vocab = cfg.vocab_size if cfg is not None else 259
-    bos = cfg.bos_token_id if cfg is not None and cfg.bos_token_id < 3 else 1
-    eos = cfg.eos_token_id if cfg is not None and cfg.eos_token_id < 3 else 2
+    bos = cfg.bos_token_id if cfg is not None and 0 <= cfg.bos_token_id < 3 else 1
+    eos = cfg.eos_token_id if cfg is not None and 0 <= cfg.eos_token_id < 3 else 2
     return ByteTokenizer(vocab_size=vocab, bos_token_id=bos, eos_token_id=eos,
                          model_max_length=(cfg.max_position_embeddings if cfg is not None else 4096))

@@ -2,7 +2,10 @@
 
 One implementation, configured by `ModelConfig`, covers Llama-3 / Mistral (RMSNorm, GQA, RoPE,
 SwiGLU, optional sliding window), Mixtral (top-k routed SwiGLU experts), GPT-2 (LayerNorm,
-learned positions, GELU, tied head) and phi-2 (parallel attn+MLP block, partial rotary, biases).
+learned positions, GELU, tied head) and phi-2 (parallel attn+MLP block, partial rotary, biases);
+designs whose layers differ from each other (`ModelConfig.layer_specs`: Vufilorn) take their layers
+from models/mixers.py and run on an fp32 residual stream, with the same embedding / cache / head /
+generation around them.
 It replaces the HF modeling code the reference runs through `AutoModelForCausalLM`
 (src/models/base_model.py:17-42) with the gfx950 op set of `..ops`:
 
@@ -28,6 +31,7 @@ from torch.utils.checkpoint import checkpoint
 
 from .. import ops
 from .config import ModelConfig
+from .mixers import Stream, build_layers
 
 
 def _param(*shape, device=None, dtype=None) -> nn.Parameter:
@@ -138,6 +142,12 @@ class Attention(nn.Module):
         return out + self.o_bias if self.o_bias is not None else out
 
 
+def _act(cfg: ModelConfig, u: torch.Tensor) -> torch.Tensor:
+    if cfg.activation == "swiglu":
+        return ops.swiglu(u)
+    return ops.relu2(u) if cfg.activation == "relu2" else ops.gelu_new(u)
+
+
 class MLP(nn.Module):
     def __init__(self, cfg: ModelConfig, device=None, dtype=None):
         super().__init__()
@@ -164,7 +174,7 @@ class MLP(nn.Module):
             if self.tp is None and self.tp_seq is None and self.down_bias is None:
                 # (no autograd, e.g. the frozen DPO reference: the same add inside the down GEMM)
                 u = ops.linear(h, self.up_proj, self.up_bias)
-                m = ops.swiglu(u) if self.cfg.activation == "swiglu" else ops.gelu_new(u)
+                m = _act(self.cfg, u)
                 return ops.linear_add(m, self.down_proj, resid)
             return self.forward(h) + resid
         seq = self.tp_seq if h.dim() == 2 else None
@@ -176,7 +186,7 @@ class MLP(nn.Module):
                 # pipelined under gate|up, the reduce-scatter behind the down GEMM chunks
                 C = tpm.tp_chunks("mlp")  # (one count for both: chunk-major rows)
                 u = tpm.sp_gather_linear(h, self.up_proj, seq, chunks=C, token_order=False)
-                m = ops.swiglu(u) if self.cfg.activation == "swiglu" else ops.gelu_new(u)
+                m = _act(self.cfg, u)
                 return tpm.sp_linear_reduce_scatter(m, self.down_proj, seq, chunks=C, token_order=False)
             h = tpm.sp_gather(h, seq)
         elif self.tp is not None:
@@ -189,7 +199,7 @@ class MLP(nn.Module):
                                       chunks=tpm.tp_chunks("mlp"))
             if tpm.TP_OVERLAP:
                 u = tpm.col_parallel_linear(h, self.up_proj, self.up_bias, self.tp)
-                m = ops.swiglu(u) if self.cfg.activation == "swiglu" else ops.gelu_new(u)
+                m = _act(self.cfg, u)
                 out = tpm.row_parallel_linear(m, self.down_proj, self.tp, chunks=tpm.tp_chunks("mlp"))
                 return out + self.down_bias if self.down_bias is not None else out
             h = tpm.tp_copy(h, self.tp)
@@ -214,7 +224,7 @@ class MLP(nn.Module):
 
             return sp_reduce_scatter(out, seq) if seq is not None else tp_reduce(out, self.tp)
         u = ops.linear(h, self.up_proj, self.up_bias)
-        m = ops.swiglu(u) if self.cfg.activation == "swiglu" else ops.gelu_new(u)
+        m = _act(self.cfg, u)
         if self.tp is None:
             return ops.linear(m, self.down_proj, self.down_bias)
         from ..parallel.tensor_parallel import sp_reduce_scatter, tp_grad_sum, tp_reduce
@@ -373,13 +383,21 @@ class CausalLM(nn.Module):
         H, V = cfg.hidden_size, cfg.vocab_size
         self.embed = _param(V, H, device=device, dtype=dtype)
         self.wpe = _param(cfg.max_position_embeddings, H, device=device, dtype=dtype) if cfg.learned_pos_emb else None
-        self.layers = nn.ModuleList([DecoderLayer(cfg, device, dtype) for _ in range(cfg.num_layers)])
+        self.schedule = cfg.layer_schedule  # [(layer index, embedding output added first)]
+        self.side_embed = None  # per-layer token input (one slice of dim token_side_dim per layer)
+        if cfg.layer_specs is not None:
+            if cfg.token_side_dim:
+                self.side_embed = _param(V, cfg.num_layers * cfg.token_side_dim, device=device, dtype=dtype)
+            self.layers = nn.ModuleList(build_layers(cfg, device, dtype))
+        else:
+            self.layers = nn.ModuleList([DecoderLayer(cfg, device, dtype) for _ in range(cfg.num_layers)])
         self.norm_w = _param(H, device=device, dtype=dtype)
         self.norm_b = _param(H, device=device, dtype=dtype) if cfg.norm_type == "layer" else None
         self.lm_head = None if (cfg.tie_word_embeddings or headless) else _param(V, H, device=device, dtype=dtype)
         self.lm_head_bias = _param(V, device=device, dtype=dtype) if (cfg.lm_head_bias and not headless) else None
         self.rope = (ops.RotaryCache(cfg.rot_dim, cfg.rope_theta, cfg.max_position_embeddings,
-                                     cfg.rope_scaling) if cfg.rot_dim > 0 else None)
+                                     cfg.rope_scaling)
+                     if cfg.rot_dim > 0 and cfg.layer_specs is None else None)
         self.gradient_checkpointing = False
         self.tp = None             # set by parallel.tensor_parallel.apply_tensor_parallel
         self.tp_size = 1
@@ -484,6 +502,8 @@ class CausalLM(nn.Module):
     def forward(self, input_ids: torch.Tensor, attention_mask: Optional[torch.Tensor] = None,
                 cache=None, segment_ids: Optional[torch.Tensor] = None) -> torch.Tensor:
         """`segment_ids` (optional, [B, T]): several sequences packed per row (see packed_layout)."""
+        if self.cfg.layer_specs is not None:
+            return self._forward_stream(input_ids, attention_mask, cache, segment_ids)
         if cache is not None:
             return self._forward_cached(input_ids, attention_mask, cache)
         sp = self.sp
@@ -530,6 +550,30 @@ class CausalLM(nn.Module):
                             self.cfg.norm_type == "rms")
         return h
 
+    def _forward_stream(self, input_ids, attention_mask, cache, segment_ids):
+        """Per-layer designs: the layer runs of `self.schedule` on an fp32 residual stream. Without a
+        cache the rows are whole sequences (a throw-away cache holds their mixers' state)."""
+        cfg = self.cfg
+        if segment_ids is not None:
+            raise NotImplementedError(f"{cfg.arch}: packed rows (segment_ids) are not supported")
+        if input_ids.is_cuda and torch.is_grad_enabled() and any(p.requires_grad for p in self.parameters()):
+            raise NotImplementedError(f"{cfg.arch}: the GPU kernels of this design are inference only; "
+                                      "run under torch.no_grad()")
+        if cache is None:
+            from .generation import KVCache
+
+            cache = KVCache(self, input_ids.shape[0], input_ids.shape[1], attention_layout(attention_mask)[0])
+        cache.reserve(cache.len + input_ids.shape[1])
+        s = Stream(ops.embed_stream(input_ids, self.embed, cfg.embed_scale))
+        x0 = s.x.clone() if any(add for _, add in self.schedule) else None
+        for j, (i, add) in enumerate(self.schedule):
+            if add:
+                s.inject = x0
+            s = self.layers[i](s, input_ids, self.side_embed, cache, cache.slots[j])
+        h = s.norm(self.norm_w, cfg.norm_eps, cfg.norm_offset, self.embed.dtype)
+        cache.step_done(input_ids.shape[1])
+        return h
+
     def sharding_engines(self) -> list:
         """The ZeRO-3 engines whose shards some of this model's layers live in."""
         out = []
@@ -570,6 +614,8 @@ class CausalLM(nn.Module):
         return h
 
     def logits(self, hidden: torch.Tensor) -> torch.Tensor:
+        if self.cfg.layer_specs is not None:
+            return ops.head_logits(hidden, self.head_weight)
         lg = None
         if self.lm_head_bias is None and self.vocab_parallel is None:
             lg = ops.decode.head_f8(hidden, self.head_weight)  # fp8 decode mode only
@@ -692,6 +738,8 @@ def init_param_tensor(cfg: ModelConfig, name: str, idx: int, shape, seed: int, d
     device = torch.device(device)
     if len(shape) == 1:
         val = 1.0 if name.endswith(("ln1_w", "ln2_w", "norm_w")) else 0.0
+        if name.endswith(("ln1_w", "ln2_w")) or name == "norm_w":
+            val -= cfg.norm_offset
         return torch.full(shape, val, device=device, dtype=dtype)
     std = cfg.init_std
     if name.endswith(("o_proj", "down_proj", "expert_down")):

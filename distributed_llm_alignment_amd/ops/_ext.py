@@ -16,42 +16,49 @@ import torch
 
 _LOCK = threading.Lock()
 _STATE = {"loaded": False, "error": None}
+_GROUPS = {"core": _STATE, "mix": {"loaded": False, "error": None}}
 # DLA_EXT_PATH: load an alternative build of the extension (A/B kernel experiments on one box)
 SO_PATH = Path(os.environ.get("DLA_EXT_PATH") or Path(__file__).resolve().parent.parent / "_C.so")
 
 
-def load(build_if_missing: bool | None = None) -> bool:
-    """Load `_C.so` once. Optionally build it first (env DLA_AUTOBUILD=1 or argument)."""
+def _so_path(group: str) -> Path:
+    return SO_PATH if group == "core" else Path(__file__).resolve().parent.parent / f"_C_{group}.so"
+
+
+def load(build_if_missing: bool | None = None, group: str = "core") -> bool:
+    """Load a group's library once (`core`: `_C.so`, `mix`: `_C_mix.so`). Optionally build it first
+    (env DLA_AUTOBUILD=1 or argument)."""
+    st, path = _GROUPS[group], _so_path(group)
     with _LOCK:
-        if _STATE["loaded"]:
+        if st["loaded"]:
             return True
         if build_if_missing is None:
             build_if_missing = os.environ.get("DLA_AUTOBUILD", "0") == "1"
         try:
-            if not SO_PATH.exists() and build_if_missing:
+            if not path.exists() and build_if_missing:
                 from .. import _build
 
-                _build.build()
-            if not SO_PATH.exists():
-                raise FileNotFoundError(str(SO_PATH))
-            torch.ops.load_library(str(SO_PATH))
-            _STATE["loaded"] = True
-            _STATE["error"] = None
+                _build.build(group=group)
+            if not path.exists():
+                raise FileNotFoundError(str(path))
+            torch.ops.load_library(str(path))
+            st["loaded"] = True
+            st["error"] = None
         except Exception as exc:  # surfaced by require()
-            _STATE["error"] = exc
-        return _STATE["loaded"]
+            st["error"] = exc
+        return st["loaded"]
 
 
-def available() -> bool:
-    return _STATE["loaded"] or load()
+def available(group: str = "core") -> bool:
+    return _GROUPS[group]["loaded"] or load(group=group)
 
 
-def require():
+def require(group: str = "core"):
     """Return the op namespace or raise loudly (GPU path must never fall back silently)."""
-    if not available():
+    if not available(group):
         raise RuntimeError(
-            "distributed_llm_alignment_amd HIP extension is not loaded "
-            f"({_STATE['error']!r}). Build it with: "
+            f"distributed_llm_alignment_amd HIP extension ({group} group) is not loaded "
+            f"({_GROUPS[group]['error']!r}). Build it with: "
             "DLA_SKIP_EXT_LOAD=1 python -m distributed_llm_alignment_amd._build"
         )
     return torch.ops.dla

@@ -34,6 +34,16 @@ class RotaryCache:
                  scaling: Optional[dict] = None):
         self.rot_dim = rot_dim
         self.theta = theta
+        self.scaling = scaling
+        self._build(max_pos)
+
+    def ensure(self, max_pos: int):
+        """Extend the tables to cover positions < max_pos (grown geometrically, new tensors)."""
+        if max_pos > self.max_pos:
+            self._build(max(max_pos, 2 * self.max_pos))
+
+    def _build(self, max_pos: int):
+        rot_dim, theta, scaling = self.rot_dim, self.theta, self.scaling
         self.max_pos = max_pos
         inv = 1.0 / (theta ** (torch.arange(0, rot_dim, 2, dtype=torch.float64) / rot_dim))
         if scaling and scaling.get("rope_type", scaling.get("type")) == "llama3":

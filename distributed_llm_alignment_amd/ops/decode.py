@@ -466,8 +466,9 @@ def refresh_folded_weights(model) -> None:
     if isinstance(hw, torch.Tensor) and getattr(hw, "_dla_f8", None) is not None:
         fp8_tiled_weight(hw)
     for layer in getattr(model, "layers", []):
-        for w, nw in ((getattr(layer.attn, "qkv_proj", None), getattr(layer, "ln1_w", None)),
-                      (getattr(layer.mlp, "up_proj", None), getattr(layer, "ln2_w", None))):
+        attn, mlp = getattr(layer, "attn", None), getattr(layer, "mlp", None)
+        for w, nw in ((getattr(attn, "qkv_proj", None), getattr(layer, "ln1_w", None)),
+                      (getattr(mlp, "up_proj", None), getattr(layer, "ln2_w", None))):
             if w is None or nw is None:
                 continue
             if getattr(w, "_dla_fold", None) is not None:
@@ -480,7 +481,7 @@ def refresh_folded_weights(model) -> None:
                 fp8_tiled_weight(w, nw)
             if getattr(w, "_dla_f8_g", None) is not None:
                 fp8_tiled_weight(w, nw, glu_il=True)
-        for w in (getattr(layer.attn, "o_proj", None), getattr(layer.mlp, "down_proj", None)):
+        for w in (getattr(attn, "o_proj", None), getattr(mlp, "down_proj", None)):
             if w is not None and getattr(w, "_dla_tile", None) is not None:
                 tiled_weight(w)
             if w is not None and getattr(w, "_dla_f8", None) is not None:
