@@ -131,3 +131,65 @@ def forward(tokens, P, cfg, layers_out=None):
         if layers_out is not None:
             layers_out.append(x)
     return (rms(x, cfg["norm"]["eps"]) * (1.0 + P["final.norm"])) @ P["embed"].T
+
+
+# ------------------------------------------------------------------ small random models for tests
+def latent(heads, dim, rot, vdim, kv_rank, q_rank, scale, size, base=10000.0):
+    return {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": kv_rank, "q_rank": q_rank,
+            "scale": scale, "rot": {"base": base, "dims": rot}, "mask": {"size": size}}
+
+
+def ret(heads, dim, vdim, rot, decay, base=10000.0):
+    return {"heads": heads, "dim": dim, "vdim": vdim, "rot": {"base": base, "dims": rot}, "decay": decay}
+
+
+def config(width, vocab, layers, side=8, scale=3.0, loop=None, eps=1e-5):
+    """layers: [(mixer dict, ff or None)]."""
+    return {"architecture": "Vufilorn", "vocab": vocab, "width": width, "embedding": {"scale": scale},
+            "norm": {"eps": eps}, "loop": loop, "token_side": {"dim": side} if side else None,
+            "layers": [{"type": "latent_attention" if "kv_rank" in m else "retention", "mixer": m,
+                        "mlp": {"kind": "dense", "ff": ff} if ff else None} for m, ff in layers]}
+
+
+def weights(cfg, seed=0, gain=1.6):
+    """Random checkpoint tensors of cfg, rounded to bfloat16 values, as float32."""
+    g = torch.Generator().manual_seed(seed)
+    P = {}
+
+    def mat(name, o, i, gn=gain):
+        P[name] = torch.randn(o, i, generator=g) * gn / math.sqrt(i)
+
+    def vec(name, n, mean):
+        P[name] = mean + 0.3 * torch.randn(n, generator=g)
+
+    H, V = cfg["width"], cfg["vocab"]
+    P["embed"] = torch.randn(V, H, generator=g) * 0.3
+    side = (cfg.get("token_side") or {}).get("dim", 0)
+    if side:
+        P["side.embed"] = torch.randn(V, len(cfg["layers"]) * side, generator=g)
+    for i, e in enumerate(cfg["layers"]):
+        m, p = e["mixer"], f"l{i}."
+        vec(p + "norm1", H, 0.0)
+        n = m["heads"]
+        if e["type"] == "latent_attention":
+            mat(p + "mix.dq", m["q_rank"], H)
+            vec(p + "mix.dq.norm", m["q_rank"], 1.0)
+            mat(p + "mix.uq", n * (m["dim"] + m["rot_dim"]), m["q_rank"])
+            mat(p + "mix.dkv", m["kv_rank"] + m["rot_dim"], H)
+            vec(p + "mix.dkv.norm", m["kv_rank"], 1.0)
+            mat(p + "mix.uk", n * m["dim"], m["kv_rank"])
+            mat(p + "mix.uv", n * m["vdim"], m["kv_rank"])
+        else:
+            for t, k in (("q", m["dim"]), ("k", m["dim"]), ("v", m["vdim"]), ("g", m["vdim"])):
+                mat(p + "mix." + t, n * k, H)
+        mat(p + "mix.o", H, n * m["vdim"])
+        if e["mlp"]:
+            vec(p + "norm2", H, 0.0)
+            mat(p + "mlp.up", e["mlp"]["ff"], H)
+            mat(p + "mlp.down", H, e["mlp"]["ff"])
+        if side:
+            mat(p + "side.gate", side, H)
+            mat(p + "side.proj", H, side)
+            vec(p + "side.norm", H, 1.0)
+    vec("final.norm", H, 0.0)
+    return {k: v.bfloat16().float() for k, v in P.items()}
