@@ -85,6 +85,8 @@ class KVCache:
         address a captured decode graph reads) in place."""
         self.len = 0
         self._pos = None
+        self.slot.zero_()  # (slot caches write a prompt at the device column too)
+        self.kv_len.fill_(1)
         self.capturing = False
         if kv_start is not None:
             self.kv_start.copy_(kv_start.to(torch.int32))
