@@ -100,6 +100,12 @@ def parse(argv=None):
                          "RCCL's stream during backward, shard AdamW, overlapped all-gather)")
     ap.add_argument("--layers", type=int, default=None, help="debug only: override layer count "
                     "(a reduced model is NOT the benchmark config)")
+    ap.add_argument("--serve", nargs="?", const="vufilorn", default=None, metavar="SIZES",
+                    help="instead of the training step: prefill / decode throughput of the per-layer design "
+                         "(vufilorn, or a comma list of presets) beside its closest attention family at equal "
+                         "size; one JSON line per size (eval/serve_bench.py)")
+    ap.add_argument("--serve-what", default="prefill,decode", help="with --serve: prefill and / or decode")
+    ap.add_argument("--serve-no-peer", action="store_true", help="with --serve: the design alone")
     a = ap.parse_args(argv)
     if a.edp_shape > 1 and a.ep_shape <= 1:
         ap.error("--edp-shape needs --ep-shape")
@@ -272,6 +278,14 @@ def main(argv=None) -> int:
     args = parse(argv)
     if args.gpus < 1:
         raise SystemExit("--gpus must be >= 1")
+    if args.serve is not None:
+        if args.gpus != 1:
+            raise SystemExit("--serve runs on one GPU")
+        from distributed_llm_alignment_amd.eval import serve_bench
+
+        serve_bench.run(serve_bench.SIZES if args.serve == "vufilorn" else args.serve.split(","),
+                        tuple(args.serve_what.split(",")), peer=not args.serve_no_peer)
+        return 0
     if "WORLD_SIZE" not in os.environ and args.gpus > 1:
         return launch_ranks(args, argv)
     env_world = int(os.environ.get("WORLD_SIZE", "1"))

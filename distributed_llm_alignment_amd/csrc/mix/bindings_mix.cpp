@@ -24,6 +24,8 @@ void launch_latent_prepare(bool, const void*, int64_t, const void*, const void*,
                            const int64_t*, const int*, const float*, const float*, int, int, int, int, int, int,
                            hipStream_t);
 int latent_prefill_waves(bool, const LatentParams&);
+bool latent_prefill_mfma_ok(const LatentParams&);
+void launch_latent_prefill_mfma(const LatentParams&, hipStream_t);
 void launch_latent_prefill_any(bool, const LatentParams&, hipStream_t);
 int latent_decode_tile(bool, const LatentParams&);
 void launch_latent_decode(bool, const LatentParams&, int, hipStream_t);
@@ -291,10 +293,14 @@ at::Tensor latent_prefill(const at::Tensor& q, const at::Tensor& kv, const at::T
   p.kv_start = starts(kv_start, q, p.B);
   p.cos_t = cos_t.data_ptr<float>();
   p.sin_t = sin_t.data_ptr<float>();
-  TORCH_CHECK(latent_prefill_waves(bf, p) > 0, "latent attention: head sizes too large");
   c10::hip::HIPGuardMasqueradingAsCUDA guard(q.device());
   auto o = at::empty({p.B, p.T, H * vdim}, q.options());
   p.o = o.data_ptr();
+  if (bf && latent_prefill_mfma_ok(p)) {
+    launch_latent_prefill_mfma(p, cur_stream(q));
+    return o;
+  }
+  TORCH_CHECK(latent_prefill_waves(bf, p) > 0, "latent attention: head sizes too large");
   launch_latent_prefill_any(bf, p, cur_stream(q));
   return o;
 }
