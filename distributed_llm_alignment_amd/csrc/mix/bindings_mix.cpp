@@ -187,9 +187,9 @@ at::Tensor retention_prefill(const at::Tensor& qkvg, int64_t H, int64_t dim, int
   TORCH_CHECK(base >= 0 && (rot == 0 || base + p.T <= cos_t.size(0)), "positions exceed the rotary table");
   c10::hip::HIPGuardMasqueradingAsCUDA guard(qkvg.device());
   auto y = at::empty({p.B, p.T, H * vdim}, qkvg.options());
-  p.y = y.data_ptr();
   p.base = base;
   p.fresh = base == 0;
+  p.y = y.data_ptr();
   p.chunk = retention_chunk(bf, p);
   if (p.chunk == 0) {
     TORCH_CHECK(2 * (dim + vdim) * 4 + 64 <= 60 * 1024, "retention: head sizes too large");

@@ -17,6 +17,11 @@
 #include "mma.h"
 
 namespace dla {
+
+bool retention_mfma_ok(const RetentionParams&);  // retention_mfma.hip
+void launch_retention_state_mfma(const RetentionParams&, hipStream_t);
+void launch_retention_output_mfma(const RetentionParams&, hipStream_t);
+
 namespace {
 
 template <typename T>
@@ -376,15 +381,19 @@ void allow_lds(K kernel, int64_t bytes) {
                               static_cast<int>(bytes));
 }
 
+void scan(const RetentionParams& p, hipStream_t st) {
+  const int64_t n = static_cast<int64_t>(p.vdim) * p.dim;
+  if (n % 4 == 0) ret_scan_kernel<4><<<dim3((n / 4 + 255) / 256, p.H, p.B), 256, 0, st>>>(p);
+  else ret_scan_kernel<1><<<dim3((n + 255) / 256, p.H, p.B), 256, 0, st>>>(p);
+}
+
 template <typename T, int VEC>
 void prefill(const RetentionParams& p, hipStream_t st) {
   const dim3 g(p.nc, p.H, p.B);
   const int64_t la = state_lds<T>(p, p.chunk), lc = output_lds<T>(p, p.chunk);
   allow_lds(ret_state_kernel<T, VEC>, la);
   ret_state_kernel<T, VEC><<<g, 256, la, st>>>(p);
-  const int64_t n = static_cast<int64_t>(p.vdim) * p.dim;
-  if (n % 4 == 0) ret_scan_kernel<4><<<dim3((n / 4 + 255) / 256, p.H, p.B), 256, 0, st>>>(p);
-  else ret_scan_kernel<1><<<dim3((n + 255) / 256, p.H, p.B), 256, 0, st>>>(p);
+  scan(p, st);
   if (p.chunk == 64) {
     allow_lds(ret_output_kernel<T, VEC, 4>, lc);
     ret_output_kernel<T, VEC, 4><<<g, 256, lc, st>>>(p);
@@ -417,11 +426,16 @@ int pick_chunk(const RetentionParams& p) {
 // chunk length of the chunked form, 0 if the recurrence takes the portion
 int retention_chunk(bool bf16, const RetentionParams& p) {
   if (p.T < 16) return 0;
+  if (bf16 && retention_mfma_ok(p)) return 128;
   return bf16 ? pick_chunk<bf16_t>(p) : pick_chunk<float>(p);
 }
 
 void launch_retention_prefill(bool bf16, const RetentionParams& p, hipStream_t st) {
-  if (bf16) {
+  if (p.chunk == 128) {  // (bf16, retention_mfma_ok)
+    launch_retention_state_mfma(p, st);
+    scan(p, st);
+    launch_retention_output_mfma(p, st);
+  } else if (bf16) {
     if (vec_ok<bf16_t>(p)) prefill<bf16_t, 8>(p, st);
     else prefill<bf16_t, 1>(p, st);
   } else {
