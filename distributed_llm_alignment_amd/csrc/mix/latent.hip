@@ -16,6 +16,10 @@
 #include "mma.h"
 
 namespace dla {
+
+bool latent_decode_mfma_ok(const LatentParams&);  // latent_decode.hip
+void launch_latent_decode_mfma(const LatentParams&, hipStream_t);
+
 namespace {
 
 constexpr float kLog2e = 1.4426950408889634f;
@@ -416,7 +420,8 @@ int64_t decode_lds(const LatentParams& p, int BN) {
 }
 
 // ------------------------------------------------------------------------------------ combine
-// grid (H, B), 256 threads: o[b][h] = W_uv[h] (sum over splits). ns <= 256.
+// grid (H, B, ceil(vdim / kCombV)), 256 threads: o[b][h] = W_uv[h] (sum over splits). ns <= 256.
+constexpr int kCombV = 32;
 template <typename T, int VEC>
 __global__ __launch_bounds__(256) void latent_combine_kernel(LatentParams p) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
@@ -426,41 +431,47 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentParams p) {
   const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
   const int64_t pb = (static_cast<int64_t>(b) * p.H + h) * p.ns;
   const float m = tid < p.ns ? p.part_ml[(pb + tid) * 2] : -INFINITY;
+  const float l0 = tid < p.ns ? p.part_ml[(pb + tid) * 2 + 1] : 0.f;
   const float mx = block_max<256>(m, scratch);
   const float w = m == -INFINITY ? 0.f : exp2f(m - mx);
-  const float l = block_sum<256>(tid < p.ns ? w * p.part_ml[(pb + tid) * 2 + 1] : 0.f, scratch);
+  const float l = block_sum<256>(w * l0, scratch);
   ws[tid] = l > 0.f ? w / l : 0.f;
   __syncthreads();
   for (int c = tid; c < p.R; c += 256) {
     float v = 0.f;
-    for (int s = 0; s < p.ns; ++s)
-      if (ws[s] != 0.f) v += ws[s] * p.part_o[(pb + s) * p.R + c];
+    int s = 0;
+    for (; s + 8 <= p.ns; s += 8) {  // (empty splits hold zeros)
+      float x[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) x[u] = p.part_o[(pb + s + u) * p.R + c];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) v += ws[s + u] * x[u];
+    }
+    for (; s < p.ns; ++s) v += ws[s] * p.part_o[(pb + s) * p.R + c];
     os[c] = v;
   }
   __syncthreads();
   const T* W = static_cast<const T*>(p.kv_up) + (static_cast<int64_t>(p.H) * p.dim + static_cast<int64_t>(h) * p.vdim) * p.R;
   T* O = static_cast<T*>(p.o) + (static_cast<int64_t>(b) * p.H + h) * p.vdim;
   const int wave = tid >> 6, lane = tid & 63;
-  constexpr int U = 4;
-  for (int v0 = wave * U; v0 < p.vdim; v0 += 4 * U) {
-    float acc[U];
+  constexpr int U = kCombV / 4;
+  const int v0 = blockIdx.z * kCombV + wave * U;
+  float acc[U];
 #pragma unroll
-    for (int u = 0; u < U; ++u) acc[u] = 0.f;
-    for (int c = lane * VEC; c < p.R; c += 64 * VEC) {
+  for (int u = 0; u < U; ++u) acc[u] = 0.f;
+  for (int c = lane * VEC; c < p.R; c += 64 * VEC) {
+    float wv[U][VEC];
 #pragma unroll
-      for (int u = 0; u < U; ++u) {
-        if (v0 + u >= p.vdim) continue;
-        float wv[VEC];
-        load_vec<T, VEC>(W + static_cast<int64_t>(v0 + u) * p.R + c, wv);
+    for (int u = 0; u < U; ++u) load_vec<T, VEC>(W + static_cast<int64_t>(min(v0 + u, p.vdim - 1)) * p.R + c, wv[u]);
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) acc[u] += wv[e] * os[c + e];
-      }
-    }
+    for (int u = 0; u < U; ++u)
 #pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const float s = wave_sum(acc[u]);
-      if (lane == 0 && v0 + u < p.vdim) O[v0 + u] = from_f<T>(s);
-    }
+      for (int e = 0; e < VEC; ++e) acc[u] += wv[u][e] * os[c + e];
+  }
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const float s = wave_sum(acc[u]);
+    if (lane == 0 && v0 + u < p.vdim) O[v0 + u] = from_f<T>(s);
   }
 }
 
@@ -483,11 +494,7 @@ void prepare(const void* down, int64_t ld, const void* qw, const void* kw, float
 }
 
 template <typename T>
-void decode(const LatentParams& p, int BN, hipStream_t st) {
-  const bool vec = p.R % 8 == 0 && reinterpret_cast<uintptr_t>(p.kv_up) % 16 == 0;
-  const dim3 ga(p.H, (p.R + 63) / 64);
-  if (vec) latent_absorb_kernel<T, 8><<<ga, 256, 0, st>>>(p);
-  else latent_absorb_kernel<T, 1><<<ga, 256, 0, st>>>(p);
+void attend_any(const LatentParams& p, int BN, hipStream_t st) {
   const int64_t lds = decode_lds<T>(p, BN);
   const dim3 gd(p.ns, (p.H + 15) / 16, p.B);
   const int nt = (p.R + 63) / 64;
@@ -501,7 +508,17 @@ void decode(const LatentParams& p, int BN, hipStream_t st) {
   else if (nt <= 8) DLA_DEC(8)
   else DLA_DEC(16)
 #undef DLA_DEC
-  const dim3 gc(p.H, p.B);
+}
+
+template <typename T>
+void decode(const LatentParams& p, int BN, hipStream_t st) {
+  const bool vec = p.R % 8 == 0 && reinterpret_cast<uintptr_t>(p.kv_up) % 16 == 0;
+  const dim3 ga(p.H, (p.R + 63) / 64);
+  if (vec) latent_absorb_kernel<T, 8><<<ga, 256, 0, st>>>(p);
+  else latent_absorb_kernel<T, 1><<<ga, 256, 0, st>>>(p);
+  if (sizeof(T) == 2 && latent_decode_mfma_ok(p)) launch_latent_decode_mfma(p, st);
+  else attend_any<T>(p, BN, st);
+  const dim3 gc(p.H, p.B, (p.vdim + kCombV - 1) / kCombV);
   if (vec) latent_combine_kernel<T, 8><<<gc, 256, 4 * p.R, st>>>(p);
   else latent_combine_kernel<T, 1><<<gc, 256, 4 * p.R, st>>>(p);
 }
