@@ -5,6 +5,7 @@
 
 #include <algorithm>
 #include <cmath>
+#include <tuple>
 
 #include "../bind_util.h"
 #include "mix_params.h"
@@ -29,6 +30,8 @@ void launch_latent_prefill_mfma(const LatentParams&, hipStream_t);
 void launch_latent_prefill_any(bool, const LatentParams&, hipStream_t);
 int latent_decode_tile(bool, const LatentParams&);
 void launch_latent_decode(bool, const LatentParams&, int, hipStream_t);
+
+void launch_stream_gemm(const StreamGemmParams&, int, hipStream_t);
 
 namespace {
 
@@ -140,6 +143,66 @@ at::Tensor relu2(const at::Tensor& u_) {
   auto y = at::empty_like(u);
   launch_relu2(bf, u.data_ptr(), y.data_ptr(), u.numel(), cur_stream(u));
   return y;
+}
+
+// Decode projection, <= 32 rows (stream_gemm.hip): epi 0 store, 1 relu^2, 2 gate, 3 stream.
+std::tuple<at::Tensor, at::Tensor> stream_gemm(const at::Tensor& a, const at::Tensor& w, int64_t epi, const OptT& ssq_in,
+                                               double eps, OptT x, const OptT& norm_w, double offset, const OptT& ids,
+                                               const OptT& table, int64_t off) {
+  check_bf16(a, "a");
+  check_bf16(w, "w");
+  same_device(a, w);
+  TORCH_CHECK(a.dim() == 2 && a.is_contiguous() && w.dim() == 2 && w.is_contiguous() && a.size(1) == w.size(1), "a [M, K], w [N, K]");
+  const int64_t M = a.size(0), N = w.size(0), K = w.size(1);
+  TORCH_CHECK(M >= 1 && M <= 32 && N >= 1 && N < (1 << 24) && K >= 8 && K < (1 << 24) && K % 8 == 0 && epi >= 0 && epi <= 3,
+              "stream_gemm: 1 <= M <= 32, K % 8 == 0");
+  check_aligned16(a, "a");
+  check_aligned16(w, "w");
+  StreamGemmParams p{};
+  p.a = cbp(a);
+  p.w = cbp(w);
+  p.M = static_cast<int>(M);
+  p.N = static_cast<int>(N);
+  p.K = static_cast<int>(K);
+  p.eps = static_cast<float>(eps);
+  p.offset = static_cast<float>(offset);
+  if (ssq_in.has_value()) {
+    check_f32(*ssq_in, "ssq_in");
+    TORCH_CHECK(ssq_in->dim() == 2 && ssq_in->size(0) == M && ssq_in->is_contiguous() && ssq_in->device() == a.device(), "ssq_in [M, blocks]");
+    p.ssq_in = ssq_in->data_ptr<float>();
+    p.nssq = static_cast<int>(ssq_in->size(1));
+  }
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(a.device());
+  auto y = at::empty({M, N}, a.options());
+  p.y = bp(y);
+  at::Tensor ssq;
+  if (epi == 3) {
+    TORCH_CHECK(x.has_value(), "stream epilogue: x");
+    check_f32(*x, "x");
+    TORCH_CHECK(x->numel() == M * N && x->size(-1) == N && x->is_contiguous() && x->device() == a.device(), "x [M, N]");
+    p.x = x->data_ptr<float>();
+    if (norm_w.has_value()) {
+      vec_like(*norm_w, a, N, "norm_w");
+      p.norm_w = cbp(*norm_w);
+    }
+    ssq = at::empty({M, (N + 15) / 16}, x->options());
+    p.ssq = ssq.data_ptr<float>();
+  } else {
+    ssq = at::empty({0}, a.options().dtype(at::kFloat));
+  }
+  if (epi == 2) {
+    TORCH_CHECK(ids.has_value() && table.has_value(), "gate epilogue: ids, table");
+    ids_ok(*ids, a, M);
+    like(*table, a, "table");
+    TORCH_CHECK(table->dim() == 2 && table->stride(1) == 1 && off >= 0 && off + N <= table->size(1), "table [V, >= off + N]");
+    p.ids = ids->data_ptr<int64_t>();
+    p.table = cbp(*table);
+    p.ldt = table->stride(0);
+    p.off = off;
+    p.vocab = table->size(0);
+  }
+  launch_stream_gemm(p, static_cast<int>(epi), cur_stream(a));
+  return {y, ssq};
 }
 
 // ---- retention ----
@@ -357,6 +420,7 @@ TORCH_LIBRARY_FRAGMENT(dla, m) {
   m.def("embed_stream(Tensor ids, Tensor table, float scale, Tensor(a!) bad) -> Tensor");
   m.def("stream_norm(Tensor(a!) x, Tensor? delta, Tensor? delta_w, Tensor? inject, Tensor? w, float eps, float offset, bool bf16) -> Tensor");
   m.def("side_gate(Tensor z, Tensor ids, Tensor table, int off) -> Tensor");
+  m.def("stream_gemm(Tensor a, Tensor w, int epi, Tensor? ssq_in, float eps, Tensor(a!)? x, Tensor? norm_w, float offset, Tensor? ids, Tensor? table, int off) -> (Tensor, Tensor)");
   m.def("relu2(Tensor u) -> Tensor");
   m.def("retention_prefill(Tensor qkvg, int H, int dim, int vdim, int rot, float eps, Tensor decay, Tensor(a!) state, Tensor? kv_start, Tensor cos, Tensor sin, int base) -> Tensor");
   m.def("retention_decode(Tensor qkvg, int H, int dim, int vdim, int rot, float eps, Tensor decay, Tensor(a!) state, Tensor slot, Tensor? kv_start, Tensor cos, Tensor sin) -> Tensor");
@@ -369,6 +433,7 @@ TORCH_LIBRARY_IMPL(dla, CUDA, m) {
   m.impl("embed_stream", &dla::embed_stream);
   m.impl("stream_norm", &dla::stream_norm);
   m.impl("side_gate", &dla::side_gate);
+  m.impl("stream_gemm", &dla::stream_gemm);
   m.impl("relu2", &dla::relu2);
   m.impl("retention_prefill", &dla::retention_prefill);
   m.impl("retention_decode", &dla::retention_decode);

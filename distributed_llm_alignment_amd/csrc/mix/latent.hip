@@ -282,6 +282,72 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentParams p) {
   }
 }
 
+// The same on MFMA (bf16, dim <= 256, dim, rot and R multiples of 8): the head's [dim, 64] piece of W_uk
+// is staged as rows in LDS and read back transposed; wave w owns 16 of the 64 columns, batch rows
+// ride on the MFMA's row dimension.
+typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
+template <int ND>
+__global__ __launch_bounds__(256) void latent_absorb_mfma_kernel(LatentParams p) {
+  constexpr int SW = 64 + 24;  // row stride: odd multiple of 16 B, 4 rows' 32-byte pieces on distinct banks
+  __shared__ __attribute__((aligned(16))) bf16_t ws[32 * ND * SW];
+  const int h = blockIdx.x, r0 = blockIdx.y * 64;
+  const int dq = p.dim + p.rot, lq = p.R + p.rot, half = p.rot >> 1;
+  const bf16_t* W = static_cast<const bf16_t*>(p.kv_up) + static_cast<int64_t>(h) * p.dim * p.R;
+  const bf16_t* Q = static_cast<const bf16_t*>(p.q) + h * dq;
+  bf16_t* out = static_cast<bf16_t*>(p.qcat) + static_cast<int64_t>(h) * lq;
+  const int64_t qsb = static_cast<int64_t>(p.H) * dq, osb = static_cast<int64_t>(p.H) * lq;
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
+  bf16x8 reg[ND];
+#pragma unroll
+  for (int j = 0; j < ND; ++j) {
+    const int i = threadIdx.x + 256 * j, d = i >> 3, c = r0 + (i & 7) * 8;
+    bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
+    if (d < p.dim && c < p.R) v = load_bf16x8(W + static_cast<int64_t>(d) * p.R + c);
+    reg[j] = v;
+  }
+  s16x8 qf[ND];
+  auto load_q = [&](int b0) {
+#pragma unroll
+    for (int k = 0; k < ND; ++k) {
+      const int d = 32 * k + 8 * g;
+      bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
+      if (d < p.dim) v = load_bf16x8(Q + min(b0 + r, p.B - 1) * qsb + d);
+      qf[k] = __builtin_bit_cast(s16x8, v);
+    }
+  };
+  load_q(0);
+#pragma unroll
+  for (int j = 0; j < ND; ++j) {
+    const int i = threadIdx.x + 256 * j;
+    store_bf16x8(ws + (i >> 3) * SW + (i & 7) * 8, reg[j]);
+  }
+  __syncthreads();
+  for (int b0 = 0; b0 < p.B; b0 += 16) {
+    if (b0) load_q(b0);
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int k = 0; k < ND; ++k) {
+      const bf16_t* wp = ws + (32 * k + 8 * g + ((lane & 15) >> 2)) * SW + 16 * wave + 4 * (lane & 3);
+      const s16x4 a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4*)(wp));
+      const s16x4 c = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4*)(wp + 4 * SW));
+      acc = Mma<bf16_t>::mma(qf[k], s16x8{a[0], a[1], a[2], a[3], c[0], c[1], c[2], c[3]}, acc);
+    }
+    const int col = r0 + 16 * wave + r;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (b0 + 4 * g + i < p.B && col < p.R) out[(b0 + 4 * g + i) * osb + col] = f2bf(acc[i]);
+  }
+  if (blockIdx.y == 0) {
+    for (int i = threadIdx.x; i < p.B * p.rot; i += 256) {
+      const int b = i / p.rot, d = i % p.rot;
+      const int64_t pos = max(min(p.slot[0], static_cast<int64_t>(p.tcap - 1)) - (p.kv_start ? p.kv_start[b] : 0), static_cast<int64_t>(0));
+      float v;
+      load_rotated<bf16_t, 1>(Q + b * qsb + p.dim, d, p.rot, p.cos_t + pos * half, p.sin_t + pos * half, &v);
+      out[b * osb + p.R + d] = f2bf(v);
+    }
+  }
+}
+
 // ------------------------------------------------------------------------------------- decode
 // grid (ns, ceil(H / 16), B), 256 threads; key tiles of BN (32 or 64); NT = latent column tiles per wave
 template <typename T, int NT>
@@ -430,6 +496,17 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentParams p) {
   __shared__ float scratch[4];
   const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
   const int64_t pb = (static_cast<int64_t>(b) * p.H + h) * p.ns;
+  // independent of everything below: the first piece of this wave's W_uv rows, the first splits
+  const T* W = static_cast<const T*>(p.kv_up) + (static_cast<int64_t>(p.H) * p.dim + static_cast<int64_t>(h) * p.vdim) * p.R;
+  const int wave = tid >> 6, lane = tid & 63;
+  constexpr int U = kCombV / 4;
+  const int v0 = blockIdx.z * kCombV + wave * U;
+  float wv[U][VEC];
+  auto load_w = [&](int c) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) load_vec<T, VEC>(W + static_cast<int64_t>(min(v0 + u, p.vdim - 1)) * p.R + c, wv[u]);
+  };
+  if (lane * VEC < p.R) load_w(lane * VEC);
   const float m = tid < p.ns ? p.part_ml[(pb + tid) * 2] : -INFINITY;
   const float l0 = tid < p.ns ? p.part_ml[(pb + tid) * 2 + 1] : 0.f;
   const float mx = block_max<256>(m, scratch);
@@ -440,29 +517,23 @@ __global__ __launch_bounds__(256) void latent_combine_kernel(LatentParams p) {
   for (int c = tid; c < p.R; c += 256) {
     float v = 0.f;
     int s = 0;
-    for (; s + 8 <= p.ns; s += 8) {  // (empty splits hold zeros)
-      float x[8];
+    for (; s + 16 <= p.ns; s += 16) {  // (empty splits hold zeros)
+      float x[16];
 #pragma unroll
-      for (int u = 0; u < 8; ++u) x[u] = p.part_o[(pb + s + u) * p.R + c];
+      for (int u = 0; u < 16; ++u) x[u] = p.part_o[(pb + s + u) * p.R + c];
 #pragma unroll
-      for (int u = 0; u < 8; ++u) v += ws[s + u] * x[u];
+      for (int u = 0; u < 16; ++u) v += ws[s + u] * x[u];
     }
     for (; s < p.ns; ++s) v += ws[s] * p.part_o[(pb + s) * p.R + c];
     os[c] = v;
   }
   __syncthreads();
-  const T* W = static_cast<const T*>(p.kv_up) + (static_cast<int64_t>(p.H) * p.dim + static_cast<int64_t>(h) * p.vdim) * p.R;
   T* O = static_cast<T*>(p.o) + (static_cast<int64_t>(b) * p.H + h) * p.vdim;
-  const int wave = tid >> 6, lane = tid & 63;
-  constexpr int U = kCombV / 4;
-  const int v0 = blockIdx.z * kCombV + wave * U;
   float acc[U];
 #pragma unroll
   for (int u = 0; u < U; ++u) acc[u] = 0.f;
   for (int c = lane * VEC; c < p.R; c += 64 * VEC) {
-    float wv[U][VEC];
-#pragma unroll
-    for (int u = 0; u < U; ++u) load_vec<T, VEC>(W + static_cast<int64_t>(min(v0 + u, p.vdim - 1)) * p.R + c, wv[u]);
+    if (c != lane * VEC) load_w(c);
 #pragma unroll
     for (int u = 0; u < U; ++u)
 #pragma unroll
@@ -514,7 +585,11 @@ template <typename T>
 void decode(const LatentParams& p, int BN, hipStream_t st) {
   const bool vec = p.R % 8 == 0 && reinterpret_cast<uintptr_t>(p.kv_up) % 16 == 0;
   const dim3 ga(p.H, (p.R + 63) / 64);
-  if (vec) latent_absorb_kernel<T, 8><<<ga, 256, 0, st>>>(p);
+  if (sizeof(T) == 2 && vec && p.dim % 8 == 0 && p.rot % 8 == 0 && p.dim <= 256 && reinterpret_cast<uintptr_t>(p.q) % 16 == 0) {
+    if (p.dim <= 64) latent_absorb_mfma_kernel<2><<<ga, 256, 0, st>>>(p);
+    else if (p.dim <= 128) latent_absorb_mfma_kernel<4><<<ga, 256, 0, st>>>(p);
+    else latent_absorb_mfma_kernel<8><<<ga, 256, 0, st>>>(p);
+  } else if (vec) latent_absorb_kernel<T, 8><<<ga, 256, 0, st>>>(p);
   else latent_absorb_kernel<T, 1><<<ga, 256, 0, st>>>(p);
   if (sizeof(T) == 2 && latent_decode_mfma_ok(p)) launch_latent_decode_mfma(p, st);
   else attend_any<T>(p, BN, st);

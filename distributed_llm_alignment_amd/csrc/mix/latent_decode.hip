@@ -13,7 +13,7 @@ namespace dla {
 namespace {
 
 constexpr float kLog2e = 1.4426950408889634f;
-constexpr int kBN = 64;
+constexpr int kBN = 64, kSS = kBN + 4, kSP = 2 * kSS;  // score row: 272 bytes (an odd multiple of 16)
 typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
 __device__ __forceinline__ s16x4 tr4(const bf16_t* p) { return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4*)(p)); }
 
@@ -22,13 +22,14 @@ __host__ __device__ constexpr int img_stride(int lp) { return lp + (2 * lp % 256
 
 // NK: 32-wide steps over kv_rank + rot, NT: 16-column latent tiles per wave
 template <int NK, int NT>
-__global__ __launch_bounds__(256) void latent_decode_mfma_kernel(LatentParams p) {
-  constexpr int SL = img_stride(32 * NK), SP = kBN + 8, NV = 4 * NK;  // NV: 16-byte chunks per row
+__global__ __launch_bounds__(256, 2) void latent_decode_mfma_kernel(LatentParams p) {
+  constexpr int SL = img_stride(32 * NK), NV = 4 * NK;  // NV: 16-byte chunks per row
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16_t* ls = reinterpret_cast<bf16_t*>(smem);
-  bf16_t* ps = ls + kBN * SL;                                // 2 planes [16][SP]
-  float* ss = reinterpret_cast<float*>(ps + 2 * 16 * SP);    // [16][kBN + 1] scores
-  float* al = ss + 16 * (kBN + 1);
+  // one row per head: 64 fp32 scores, overwritten in place by their weights' planes (64 hi, 64 lo)
+  bf16_t* ps = ls + kBN * SL;
+  float* ss = reinterpret_cast<float*>(ps);
+  float* al = ss + 16 * kSS;
   const int split = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
   const int lq = p.R + p.rot, nh = min(16, p.H - h0);
@@ -81,11 +82,12 @@ __global__ __launch_bounds__(256) void latent_decode_mfma_kernel(LatentParams p)
       s = Mma<bf16_t>::mma(qf[k], Mma<bf16_t>::row(ls + (16 * wave + r) * SL + 32 * k + 8 * g), s);
 #pragma unroll
     for (int i = 0; i < 4; ++i)
-      ss[(4 * g + i) * (kBN + 1) + 16 * wave + r] = 16 * wave + r < cnt ? s[i] * (p.scale * kLog2e) : -INFINITY;
+      ss[(4 * g + i) * kSS + 16 * wave + r] = 16 * wave + r < cnt ? s[i] * (p.scale * kLog2e) : -INFINITY;
     __syncthreads();
     {
-      const float* row = ss + (4 * wave + g) * (kBN + 1) + r;
+      const float* row = ss + (4 * wave + g) * kSS + r;
       const float x[4] = {row[0], row[16], row[32], row[48]};
+      __builtin_amdgcn_wave_barrier();  // (a row's 16 lanes have read it before any of them writes)
       float mx = fmaxf(fmaxf(x[0], x[1]), fmaxf(x[2], x[3]));
 #pragma unroll
       for (int o = 1; o < 16; o <<= 1) mx = fmaxf(mx, __shfl_xor(mx, o, 64));
@@ -97,7 +99,7 @@ __global__ __launch_bounds__(256) void latent_decode_mfma_kernel(LatentParams p)
       for (int j = 0; j < 4; ++j) {
         const float e = exp2f(x[j] - mu);
         l += e;
-        put_planes<bf16_t>(ps + (4 * wave + g) * SP + 16 * j + r, 16 * SP, e);
+        put_planes<bf16_t>(ps + (4 * wave + g) * kSP + 16 * j + r, kBN, e);
       }
 #pragma unroll
       for (int o = 1; o < 16; o <<= 1) l += __shfl_xor(l, o, 64);
@@ -108,8 +110,8 @@ __global__ __launch_bounds__(256) void latent_decode_mfma_kernel(LatentParams p)
     s16x8 ph[2], pl[2];
 #pragma unroll
     for (int k = 0; k < 2; ++k) {
-      ph[k] = Mma<bf16_t>::row(ps + r * SP + 32 * k + 8 * g);
-      pl[k] = Mma<bf16_t>::row(ps + (16 + r) * SP + 32 * k + 8 * g);
+      ph[k] = Mma<bf16_t>::row(ps + r * kSP + 32 * k + 8 * g);
+      pl[k] = Mma<bf16_t>::row(ps + r * kSP + kBN + 32 * k + 8 * g);
     }
     float a4[4];
 #pragma unroll
@@ -146,7 +148,7 @@ __global__ __launch_bounds__(256) void latent_decode_mfma_kernel(LatentParams p)
 
 template <int NK, int NT>
 void go(const LatentParams& p, hipStream_t st) {
-  constexpr int lds = 2 * (kBN * img_stride(32 * NK) + 2 * 16 * (kBN + 8)) + 4 * (16 * (kBN + 1) + 16);
+  constexpr int lds = 2 * kBN * img_stride(32 * NK) + 4 * (16 * kSS + 16);
   if (lds > 64 * 1024)
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(latent_decode_mfma_kernel<NK, NT>),
                               hipFuncAttributeMaxDynamicSharedMemorySize, lds);

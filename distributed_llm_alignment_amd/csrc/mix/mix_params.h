@@ -47,4 +47,21 @@ struct LatentParams {
   int tcap;               // decode: cache rows
 };
 
+struct StreamGemmParams {
+  const uint16_t* a;       // [M, K] bf16 contiguous
+  const uint16_t* w;       // [N, K] bf16 contiguous
+  uint16_t* y;             // [M, N]
+  int M, N, K;
+  const float* ssq_in;     // [M, nssq] partial sums of squares of a's rows before the norm weight, or nullptr
+  int nssq;
+  float eps;
+  float* x;                // stream epilogue: fp32 [M, N], updated in place
+  const uint16_t* norm_w;  // stream epilogue: the next norm's weight, or nullptr
+  float offset;
+  float* ssq;              // stream epilogue: [M, ceil(N / 16)]
+  const int64_t* ids;      // gate epilogue: [M]
+  const uint16_t* table;
+  int64_t ldt, off, vocab;
+};
+
 }  // namespace dla
