@@ -2,8 +2,8 @@
 // fp32: latent.hip).
 //
 // Workgroup = (key split, group of 16 heads, sequence), 4 waves. A tile of 64 cache rows is read once
-// for all heads (16-byte loads, the whole tile in flight, the next tile in flight behind the
-// compute), kept as one row image in LDS and used twice: as keys along its rows (wave w: 16 of the
+// for all heads, straight into LDS (LDS-DMA, the whole tile in flight, no registers), kept as one
+// XOR-swizzled row image and used twice: as keys along its rows (wave w: 16 of the
 // 64 keys against the 16 heads) and as values along its columns by transposed reads (wave w: every
 // fourth 16-column tile of the latent). Softmax weights are fp32, in the product as hi + lo planes.
 #include "mix_params.h"
@@ -17,17 +17,21 @@ constexpr int kBN = 64, kSS = kBN + 4, kSP = 2 * kSS;  // score row: 272 bytes (
 typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
 __device__ __forceinline__ s16x4 tr4(const bf16_t* p) { return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4*)(p)); }
 
-// row stride (elements): odd multiple of 16 B, and 4 consecutive rows' 32-byte pieces on distinct banks
-__host__ __device__ constexpr int img_stride(int lp) { return lp + (2 * lp % 256 == 0 ? 24 : 8); }
+// Position of 16-byte chunk c of row n in the image (rows of NV = 8 (mod 16) chunks). The XOR inside
+// aligned groups of 8 chunks spreads both a column of 16 rows (score fragments) and 4 rows x 32 bytes
+// (transposed reads) over all banks.
+__device__ __forceinline__ int img_f(int n) { return ((n >> 1) & 1) << 1 | ((n >> 2) & 1) << 2 | ((n >> 3) & 1); }
+template <int NV>
+__device__ __forceinline__ int img(int n, int c) { return (n * NV + (c ^ img_f(n))) * 8; }
 
 // NK: 32-wide steps over kv_rank + rot, NT: 16-column latent tiles per wave
 template <int NK, int NT>
 __global__ __launch_bounds__(256, 2) void latent_decode_mfma_kernel(LatentParams p) {
-  constexpr int SL = img_stride(32 * NK), NV = 4 * NK;  // NV: 16-byte chunks per row
+  constexpr int NV = 4 * NK;  // 16-byte chunks per row
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   bf16_t* ls = reinterpret_cast<bf16_t*>(smem);
   // one row per head: 64 fp32 scores, overwritten in place by their weights' planes (64 hi, 64 lo)
-  bf16_t* ps = ls + kBN * SL;
+  bf16_t* ps = ls + kBN * 8 * NV;
   float* ss = reinterpret_cast<float*>(ps);
   float* al = ss + 16 * kSS;
   const int split = blockIdx.x, h0 = blockIdx.y * 16, b = blockIdx.z;
@@ -40,14 +44,14 @@ __global__ __launch_bounds__(256, 2) void latent_decode_mfma_kernel(LatentParams
   per = (per + kBN - 1) / kBN * kBN;
   const int k0 = lo + split * per, k1 = min(k0 + per, newest + 1);
   const bf16_t* L = static_cast<const bf16_t*>(p.latent) + b * p.l_sb;
-  bf16x8 reg[NK];
   auto load_tile = [&](int c0) {
 #pragma unroll
     for (int j = 0; j < NK; ++j) {
-      const int i = threadIdx.x + 256 * j, n = i / NV, d = (i % NV) * 8;
-      bf16x8 v = {0, 0, 0, 0, 0, 0, 0, 0};
-      if (d < lq) v = load_bf16x8(L + static_cast<int64_t>(min(c0 + n, k1 - 1)) * p.l_st + d);
-      reg[j] = v;
+      const int i0 = 256 * j + 64 * wave, i = i0 + lane, n = i / NV;
+      const int c = (i % NV) ^ img_f(n);  // source chunk of this position; past the row: any (times q = 0)
+      const bf16_t* src = L + static_cast<int64_t>(min(c0 + n, k1 - 1)) * p.l_st + (8 * c < lq ? 8 * c : 0);
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
+                                       (__attribute__((address_space(3))) void*)(ls + 8 * i0), 16, 0, 0);
     }
   };
   if (k0 < k1) load_tile(k0);
@@ -68,18 +72,16 @@ __global__ __launch_bounds__(256, 2) void latent_decode_mfma_kernel(LatentParams
   float m_run = -INFINITY, l_run = 0.f;  // of head 4 wave + g
   for (int c0 = k0; c0 < k1; c0 += kBN) {
     const int cnt = min(kBN, k1 - c0);
-    __syncthreads();
-#pragma unroll
-    for (int j = 0; j < NK; ++j) {
-      const int i = threadIdx.x + 256 * j;
-      store_bf16x8(ls + (i / NV) * SL + (i % NV) * 8, reg[j]);
+    if (c0 != k0) {
+      __syncthreads();  // every wave is done with the last tile
+      load_tile(c0);
     }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     __syncthreads();
-    if (c0 + kBN < k1) load_tile(c0 + kBN);
     f32x4 s = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int k = 0; k < NK; ++k)
-      s = Mma<bf16_t>::mma(qf[k], Mma<bf16_t>::row(ls + (16 * wave + r) * SL + 32 * k + 8 * g), s);
+      s = Mma<bf16_t>::mma(qf[k], Mma<bf16_t>::row(ls + img<NV>(16 * wave + r, 4 * k + g)), s);
 #pragma unroll
     for (int i = 0; i < 4; ++i)
       ss[(4 * g + i) * kSS + 16 * wave + r] = 16 * wave + r < cnt ? s[i] * (p.scale * kLog2e) : -INFINITY;
@@ -123,8 +125,8 @@ __global__ __launch_bounds__(256, 2) void latent_decode_mfma_kernel(LatentParams
       for (int i = 0; i < 4; ++i) acc[t][i] *= a4[i];
 #pragma unroll
       for (int k = 0; k < 2; ++k) {
-        const bf16_t* vp = ls + (32 * k + 8 * g + ((lane & 15) >> 2)) * SL + v0 + 4 * (lane & 3);
-        const s16x4 a = tr4(vp), c = tr4(vp + 4 * SL);
+        const int n = 32 * k + 8 * g + ((lane & 15) >> 2), ch = (v0 >> 3) + ((lane & 3) >> 1);
+        const s16x4 a = tr4(ls + img<NV>(n, ch) + 4 * (lane & 1)), c = tr4(ls + img<NV>(n + 4, ch) + 4 * (lane & 1));
         const s16x8 bv = {a[0], a[1], a[2], a[3], c[0], c[1], c[2], c[3]};
         acc[t] = Mma<bf16_t>::mma(ph[k], bv, acc[t]);
         acc[t] = Mma<bf16_t>::mma(pl[k], bv, acc[t]);
@@ -148,7 +150,7 @@ __global__ __launch_bounds__(256, 2) void latent_decode_mfma_kernel(LatentParams
 
 template <int NK, int NT>
 void go(const LatentParams& p, hipStream_t st) {
-  constexpr int lds = 2 * kBN * img_stride(32 * NK) + 4 * (16 * kSS + 16);
+  constexpr int lds = 2 * kBN * 32 * NK + 4 * (16 * kSS + 16);
   if (lds > 64 * 1024)
     (void)hipFuncSetAttribute(reinterpret_cast<const void*>(latent_decode_mfma_kernel<NK, NT>),
                               hipFuncAttributeMaxDynamicSharedMemorySize, lds);
