@@ -93,7 +93,7 @@ def _layer_map(cfg, i: int) -> List[Tuple[str, str, tuple]]:
                   (n + "mix.kv_up", p + "mix.uk", (0, k)), (n + "mix.kv_up", p + "mix.uv", (k, v))]
         else:
             k, v = x["heads"] * x["dim"], x["heads"] * x["vdim"]
-            m += [(n + "mix.qkvg_proj", p + "mix." + t, (a, b)) for t, a, b in
+            m += [(n + "mix.in_proj", p + "mix." + t, (a, b)) for t, a, b in
                   (("q", 0, k), ("k", k, 2 * k), ("v", 2 * k, 2 * k + v), ("g", 2 * k + v, 2 * (k + v)))]
         m.append((n + "mix.o_proj", p + "mix.o", None))
         if spec.get("mlp"):

@@ -34,12 +34,11 @@ class Stream:
     delta: Optional[torch.Tensor] = None
     delta_w: Optional[torch.Tensor] = None  # plain RMS norm of delta with this weight before the add
     inject: Optional[torch.Tensor] = None
-    ssq: Optional[torch.Tensor] = None      # decode: partial sums of squares of x's rows
 
     def norm(self, w, eps: float, offset: float, dtype) -> torch.Tensor:
         """Fold the pending update into x and return the normed rows."""
         y, self.x = ops.stream_norm(self.x, self.delta, self.delta_w, self.inject, w, eps, offset, dtype)
-        self.delta = self.delta_w = self.inject = self.ssq = None
+        self.delta = self.delta_w = self.inject = None
         return y
 
     def cast(self, eps: float, dtype) -> torch.Tensor:
@@ -107,14 +106,14 @@ class LatentAttention(nn.Module):
         return CacheSlot(self.rope, max_len, device, latent=torch.zeros(
             (batch, max_len, self.kv_rank + self.rot), device=device, dtype=dtype))
 
-    def attend(self, down: torch.Tensor, cache, slot: CacheSlot) -> torch.Tensor:
+    def mix(self, down: torch.Tensor, cache, slot: CacheSlot, lin=ops.stream_linear) -> torch.Tensor:
         """down = in_proj output [B, T, q_rank + kv_rank + rot] -> heads' outputs [B, T, heads * vdim];
         the new tokens' latents go into the slot."""
-        B, T, _ = down.shape
+        _, T, _ = down.shape
         latent = slot.t["latent"]
         cq = ops.latent.prepare(down, self.q_norm_w, self.kv_norm_w, self.eps, latent, cache.slot,
                                 cache.kv_start, slot.cos, slot.sin, base=cache.len)
-        q = ops.stream_linear(cq, self.q_up)
+        q = lin(cq, self.q_up)
         if T == 1 and cache.len > 0:
             return ops.latent.decode(q, latent, self.kv_up, self.heads, self.dim, self.rot, self.vdim,
                                      self.scale, self.window, cache.slot, cache.kv_start, slot.cos,
@@ -129,8 +128,10 @@ class LatentAttention(nn.Module):
                                   q_base=cache.len, k_base=lo)
 
     def forward(self, h, cache, slot):
-        a = self.attend(ops.stream_linear(h, self.in_proj), cache, slot)
-        return ops.stream_linear(a, self.o_proj)
+        return ops.stream_linear(self.mix(ops.stream_linear(h, self.in_proj), cache, slot), self.o_proj)
+
+    def matrices(self):
+        return (self.in_proj, self.q_up, self.o_proj)
 
 
 class Retention(nn.Module):
@@ -146,7 +147,7 @@ class Retention(nn.Module):
         self.decay = [float(x) for x in m["decay"]]
         self._decay = {}
         # rows [q; k; v; g]
-        self.qkvg_proj = _param(2 * self.heads * (self.dim + self.vdim), H, device=device, dtype=dtype)
+        self.in_proj = _param(2 * self.heads * (self.dim + self.vdim), H, device=device, dtype=dtype)
         self.o_proj = _param(H, self.heads * self.vdim, device=device, dtype=dtype)
 
     def decays(self, device) -> torch.Tensor:
@@ -162,8 +163,8 @@ class Retention(nn.Module):
         return CacheSlot(self.rope, max_len, device, state=torch.zeros(
             (batch, self.heads, self.vdim, self.dim), device=device, dtype=torch.float32))
 
-    def mix(self, qkvg: torch.Tensor, cache, slot: CacheSlot) -> torch.Tensor:
-        B, T, _ = qkvg.shape
+    def mix(self, qkvg: torch.Tensor, cache, slot: CacheSlot, lin=None) -> torch.Tensor:
+        _, T, _ = qkvg.shape
         args = (self.heads, self.dim, self.vdim, self.rope_key[0], self.eps, self.decays(qkvg.device),
                 slot.t["state"], cache.slot, cache.kv_start, slot.cos, slot.sin)
         if T == 1 and cache.len > 0:
@@ -171,7 +172,10 @@ class Retention(nn.Module):
         return ops.retention.prefill(qkvg, *args, base=cache.len)
 
     def forward(self, h, cache, slot):
-        return ops.stream_linear(self.mix(ops.stream_linear(h, self.qkvg_proj), cache, slot), self.o_proj)
+        return ops.stream_linear(self.mix(ops.stream_linear(h, self.in_proj), cache, slot), self.o_proj)
+
+    def matrices(self):
+        return (self.in_proj, self.o_proj)
 
 
 MIXERS = {"latent_attention": LatentAttention, "retention": Retention}
@@ -206,8 +210,35 @@ class StreamLayer(nn.Module):
         self.side = TokenSide(cfg, device, dtype) if cfg.token_side_dim else None
         self.recompute = None
 
+    def fused_ok(self, rows: int) -> bool:
+        """A decode step of this layer can run on the fused projections (norm in front, stream add /
+        activation / gate behind)."""
+        ws = self.mix.matrices()
+        if self.mlp is not None:
+            ws += (self.mlp.up_proj, self.mlp.down_proj)
+        if self.side is not None:
+            ws += (self.side.gate, self.side.proj)
+        return ops.stream.fused_ok(rows, self.ln1_w.dtype, *ws)
+
+    def decode_fused(self, s: Stream, ids: torch.Tensor, side_embed, cache, slot: CacheSlot) -> Stream:
+        cfg, st = self.cfg, ops.stream
+        eps, off = cfg.norm_eps, cfg.norm_offset
+        h = s.norm(self.ln1_w, eps, off, self.ln1_w.dtype)
+        a = self.mix.mix(st.fused_linear(h, self.mix.in_proj), cache, slot, st.fused_linear)
+        # each add hands the next reader of x its rows: weighted for a norm, plain for the side gate
+        h, ssq = st.fused_add(a, self.mix.o_proj, s.x, self.ln2_w if self.mlp is not None else None, off)
+        if self.mlp is not None:
+            m = st.fused_linear(h, self.mlp.up_proj, ssq, eps, relu2=True)
+            h, _ = st.fused_add(m, self.mlp.down_proj, s.x, None, 0.0)
+        if self.side is not None:
+            g = st.fused_gate(h, self.side.gate, ids, side_embed, self.index * cfg.token_side_dim)
+            s.delta, s.delta_w = st.fused_linear(g, self.side.proj), self.side.norm_w
+        return s
+
     def forward(self, s: Stream, ids: torch.Tensor, side_embed, cache, slot: CacheSlot) -> Stream:
         cfg, dt = self.cfg, self.ln1_w.dtype
+        if ids.shape[1] == 1 and not torch.is_grad_enabled() and self.fused_ok(ids.shape[0]):
+            return self.decode_fused(s, ids, side_embed, cache, slot)
         h = s.norm(self.ln1_w, cfg.norm_eps, cfg.norm_offset, dt)
         s.delta = self.mix(h, cache, slot)
         if self.mlp is not None:

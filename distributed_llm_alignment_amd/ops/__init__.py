@@ -1,6 +1,6 @@
 """gfx950 compute ops. GPU tensors run the in-tree HIP kernels (`torch.ops.dla.*`); CPU tensors
 run the pure-PyTorch references (test tier / numerics oracles)."""
-from . import _ext, decode, latent, moe, retention
+from . import _ext, decode, latent, moe, retention, stream
 from .embedding import embedding
 from .activations import gelu_new, swiglu, swiglu_mlp, swiglu_mlp_ok
 from .attention import RotaryCache, attention_core, qkv_attention, ref_attention
@@ -18,6 +18,6 @@ __all__ = [
     "ref_attention", "linear_logprob", "seq_reduce", "sequence_logprob", "shifted_targets",
     "token_nll", "dpo_loss", "ensemble_kl", "kl_penalty_pg", "pairwise_loss", "gae",
     "ppo_policy_loss", "ppo_value_loss", "add_norm", "layer_norm", "rms_norm", "linear", "linear_add",
-    "accumulate_weight_grad", "latent", "retention", "embed_stream", "head_logits", "relu2", "side_gate",
+    "accumulate_weight_grad", "latent", "retention", "stream", "embed_stream", "head_logits", "relu2", "side_gate",
     "stream_linear", "stream_norm",
 ]

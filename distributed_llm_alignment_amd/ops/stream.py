@@ -7,6 +7,7 @@ fp32 compute dtypes run the same kernels. CPU tensors use the PyTorch forms belo
 """
 from __future__ import annotations
 
+import os
 from typing import Optional, Tuple
 
 import torch
@@ -70,4 +71,49 @@ def stream_linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
 
 
 def head_logits(h: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+    rows = h.numel() // h.shape[-1]
+    if h.is_cuda and fused_ok(rows, h.dtype, w) and not torch.is_grad_enabled():
+        return fused_linear(h, w)
     return F.linear(h, w)
+
+
+# ------------------------------------------------------------------------ fused decode projections
+# (csrc/mix/stream_gemm.hip) few rows: the norm before a projection and the stream add / activation /
+# gate behind it run inside the projection's launch. DLA_STREAM_FUSED=0: library GEMMs + the kernels above.
+STREAM_FUSED = os.environ.get("DLA_STREAM_FUSED", "1") != "0"
+STREAM_FUSED_ROWS = int(os.environ.get("DLA_STREAM_FUSED_ROWS", "32"))
+_STORE, _RELU2, _GATE, _STREAM = range(4)
+
+
+def fused_ok(rows: int, dtype: torch.dtype, *weights: torch.Tensor) -> bool:
+    """These projections can run on the fused decode kernel (bf16, GPU, <= 32 rows, K % 8 == 0)."""
+    return (STREAM_FUSED and 1 <= rows <= min(STREAM_FUSED_ROWS, 32) and dtype == torch.bfloat16
+            and all(w.is_cuda and w.dim() == 2 and w.is_contiguous() and w.shape[1] % 8 == 0 and w.data_ptr() % 16 == 0
+                    for w in weights))
+
+
+def _rows(a: torch.Tensor) -> torch.Tensor:
+    return a.reshape(-1, a.shape[-1]).contiguous()
+
+
+def fused_linear(a: torch.Tensor, w: torch.Tensor, ssq: Optional[torch.Tensor] = None, eps: float = 0.0,
+                 relu2: bool = False) -> torch.Tensor:
+    """rowscale * (a W^T) [then relu(.)^2]; `ssq`: partial sums of squares from `fused_add` (rowscale =
+    rsqrt(mean + eps)), None: no scale."""
+    y, _ = _ext.require("mix").stream_gemm(_rows(a), w, _RELU2 if relu2 else _STORE, ssq, float(eps), None, None, 0.0,
+                                           None, None, 0)
+    return y.view(*a.shape[:-1], w.shape[0])
+
+
+def fused_gate(a: torch.Tensor, w: torch.Tensor, ids: torch.Tensor, side_embed: torch.Tensor, off: int) -> torch.Tensor:
+    """side_gate(a W^T, ids, side_embed, off)."""
+    y, _ = _ext.require("mix").stream_gemm(_rows(a), w, _GATE, None, 0.0, None, None, 0.0, ids.contiguous(), side_embed,
+                                           int(off))
+    return y.view(*a.shape[:-1], w.shape[0])
+
+
+def fused_add(a: torch.Tensor, w: torch.Tensor, x: torch.Tensor, norm_w: Optional[torch.Tensor], offset: float):
+    """x += a W^T (fp32, in place). Returns (x * (offset + norm_w), or x, in bf16; x's partial sums of
+    squares): what the next projection needs to see RMSNorm(x)."""
+    y, ssq = _ext.require("mix").stream_gemm(_rows(a), w, _STREAM, None, 0.0, x, norm_w, float(offset), None, None, 0)
+    return y.view(*a.shape[:-1], w.shape[0]), ssq

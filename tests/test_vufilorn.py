@@ -254,6 +254,33 @@ def test_embedding_side_gate_relu2(where):
     rel(ops.relu2(u), torch.relu(u.double().cpu()) ** 2, where)
 
 
+@GPU
+@pytest.mark.parametrize("M", [1, 5, 16, 17, 32])
+@pytest.mark.parametrize("N,K", [(50, 72), (256, 2048), (96, 8), (2048, 8192), (33, 264)])
+def test_fused_decode_projections(M, N, K):
+    """Every epilogue against float64, with and without the row scale."""
+    where = ("cuda", torch.bfloat16)
+    a, w = rnd(where, M, 1, K), rnd(where, N, K, scale=K ** -0.5)
+    st, f = ops.stream, lambda t: t.double().cpu()  # noqa: E731
+    want = f(a)[:, 0] @ f(w).T
+    rel(st.fused_linear(a, w)[:, 0], want, where)
+    ssq = torch.rand(M, 7, device="cuda") + 0.1
+    scale = 1 / torch.sqrt(f(ssq).sum(1, keepdim=True) / K + 1e-3)
+    rel(st.fused_linear(a, w, ssq, 1e-3)[:, 0], want * scale, where)
+    rel(st.fused_linear(a, w, ssq, 1e-3, relu2=True)[:, 0], torch.relu(want * scale) ** 2, where)
+    table = rnd(where, 30, N + 12)
+    ids = torch.randint(0, 30, (M, 1), device="cuda")
+    rel(st.fused_gate(a, w, ids, table, 8)[:, 0], O.gelu_tanh(want) * f(table)[ids.cpu()[:, 0], 8:8 + N], where)
+    x, nw = torch.randn(M, 1, N, device="cuda"), rnd(where, N)
+    xw = f(x)[:, 0] + want
+    for weight in (nw, None):
+        xi = x.clone()
+        h, sq = st.fused_add(a, w, xi, weight, 1.0)
+        rel(xi[:, 0], xw, where, b16=2e-5)  # the stream is fp32
+        rel(sq.sum(1), (xw ** 2).sum(1), where, b16=2e-5)
+        rel(h[:, 0], xw if weight is None else xw * (1 + f(weight)), where)
+
+
 @pytest.mark.parametrize("where", FP32)
 def test_embedding_out_of_range(where):
     if where[0] == "cpu":
