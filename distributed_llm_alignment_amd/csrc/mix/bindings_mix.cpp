@@ -238,6 +238,7 @@ RetentionParams retention_params(const at::Tensor& qkvg, int64_t H, int64_t dim,
   p.vdim = static_cast<int>(vdim);
   p.rot = static_cast<int>(rot);
   p.eps = static_cast<float>(eps);
+  p.vsplit = 1;
   p.kscale = 1.f / std::sqrt(static_cast<float>(dim));
   return p;
 }
@@ -268,7 +269,7 @@ at::Tensor retention_prefill(const at::Tensor& qkvg, int64_t H, int64_t dim, int
 
 at::Tensor retention_decode(const at::Tensor& qkvg, int64_t H, int64_t dim, int64_t vdim, int64_t rot, double eps,
                             const at::Tensor& decay, at::Tensor state, const at::Tensor& slot, const OptT& kv_start,
-                            const at::Tensor& cos_t, const at::Tensor& sin_t) {
+                            const at::Tensor& cos_t, const at::Tensor& sin_t, const OptT& cnt) {
   RetentionParams p = retention_params(qkvg, H, dim, vdim, rot, eps, decay, state, kv_start, cos_t, sin_t);
   TORCH_CHECK(p.T == 1, "retention_decode: one token per row");
   TORCH_CHECK(2 * (dim + vdim) * 4 + 64 <= 60 * 1024, "retention: head sizes too large");
@@ -276,6 +277,21 @@ at::Tensor retention_decode(const at::Tensor& qkvg, int64_t H, int64_t dim, int6
   auto y = at::empty({p.B, 1, H * vdim}, qkvg.options());
   p.y = y.data_ptr();
   p.slot = slot_ptr(slot, qkvg);
+  // few (sequence, head) pairs with a large state (>= 128 KB): several workgroups share the value rows
+  // of one pair, >= 32 rows each (smaller states lose more to the hand-off than they gain)
+  at::Tensor part;
+  if (cnt.has_value() && dim * vdim >= 32 * 1024) {
+    check_i32(*cnt, "cnt");
+    TORCH_CHECK(cnt->is_contiguous() && cnt->numel() >= p.B * H && cnt->device() == qkvg.device(), "cnt int32, >= B H");
+    int64_t vs = std::min<int64_t>(512 / std::max<int64_t>(1, p.B * H), vdim / 32);
+    vs = std::min<int64_t>(vs, 8);
+    if (vs > 1) {
+      part = at::empty({p.B, H, vdim}, state.options());
+      p.osplit = part.data_ptr<float>();
+      p.cnt = cnt->data_ptr<int>();
+      p.vsplit = static_cast<int>(vs);
+    }
+  }
   launch_retention_recurrent(qkvg.scalar_type() == at::kBFloat16, p, cur_stream(qkvg));
   return y;
 }
@@ -423,7 +439,7 @@ TORCH_LIBRARY_FRAGMENT(dla, m) {
   m.def("stream_gemm(Tensor a, Tensor w, int epi, Tensor? ssq_in, float eps, Tensor(a!)? x, Tensor? norm_w, float offset, Tensor? ids, Tensor? table, int off) -> (Tensor, Tensor)");
   m.def("relu2(Tensor u) -> Tensor");
   m.def("retention_prefill(Tensor qkvg, int H, int dim, int vdim, int rot, float eps, Tensor decay, Tensor(a!) state, Tensor? kv_start, Tensor cos, Tensor sin, int base) -> Tensor");
-  m.def("retention_decode(Tensor qkvg, int H, int dim, int vdim, int rot, float eps, Tensor decay, Tensor(a!) state, Tensor slot, Tensor? kv_start, Tensor cos, Tensor sin) -> Tensor");
+  m.def("retention_decode(Tensor qkvg, int H, int dim, int vdim, int rot, float eps, Tensor decay, Tensor(a!) state, Tensor slot, Tensor? kv_start, Tensor cos, Tensor sin, Tensor(b!)? cnt) -> Tensor");
   m.def("latent_prepare(Tensor down, Tensor q_norm_w, Tensor kv_norm_w, float eps, Tensor(a!) latent, Tensor slot, Tensor? kv_start, Tensor cos, Tensor sin) -> Tensor");
   m.def("latent_prefill(Tensor q, Tensor kv, Tensor kr, int H, int dim, int rot, int vdim, float scale, int window, Tensor? kv_start, Tensor cos, Tensor sin, int q_base, int k_base) -> Tensor");
   m.def("latent_decode(Tensor q, Tensor latent, Tensor kv_up, int H, int dim, int rot, int vdim, float scale, int window, Tensor slot, Tensor? kv_start, Tensor cos, Tensor sin) -> Tensor");

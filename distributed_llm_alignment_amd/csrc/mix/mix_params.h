@@ -19,6 +19,9 @@ struct RetentionParams {
   int B, T, H, dim, vdim, rot;
   float eps, kscale;
   int chunk, nc;
+  float* osplit;          // decode split: [B, H, vdim] unnormalised outputs
+  int* cnt;               // decode split: arrival counters [B, H], zero between launches
+  int vsplit;             // decode split: workgroups per (sequence, head)
   int npos;               // rows of the rotary tables
   int fresh;              // the state starts at zero (base == 0)
 };

@@ -93,13 +93,17 @@ __device__ __forceinline__ void put_planes<bf16_t>(bf16_t* p, int plane, float v
 template <>
 __device__ __forceinline__ void put_planes<float>(float* p, int, float v) { p[0] = v; }
 
-// VEC consecutive elements -> fp32 (16-byte loads when VEC == 8; the caller checks alignment)
+// VEC consecutive elements -> fp32 (8- or 16-byte loads; the caller checks alignment)
 template <typename T, int VEC>
 __device__ __forceinline__ void load_vec(const T* p, float* o) {
   if constexpr (VEC == 8 && sizeof(T) == 2) {
     const bf16x8 v = load_bf16x8(reinterpret_cast<const bf16_t*>(p));
 #pragma unroll
     for (int j = 0; j < 8; ++j) o[j] = bf2f(v[j]);
+  } else if constexpr (VEC == 4 && sizeof(T) == 2) {
+    const bf16x4 v = *reinterpret_cast<const bf16x4*>(p);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = bf2f(v[j]);
   } else if constexpr (VEC % 4 == 0 && sizeof(T) == 4) {
 #pragma unroll
     for (int j = 0; j < VEC; j += 4) {
@@ -116,6 +120,9 @@ template <typename T, int VEC>
 __device__ __forceinline__ void store_vec(T* p, const float* v) {
   if constexpr (VEC == 8 && sizeof(T) == 2) {
     store_bf16x8(reinterpret_cast<bf16_t*>(p), pack_bf16x8(v));
+  } else if constexpr (VEC == 4 && sizeof(T) == 2) {
+    typedef uint32_t u32x2 __attribute__((ext_vector_type(2)));
+    *reinterpret_cast<u32x2*>(p) = u32x2{pack2bf(v[0], v[1]), pack2bf(v[2], v[3])};
   } else if constexpr (VEC % 4 == 0 && sizeof(T) == 4) {
 #pragma unroll
     for (int j = 0; j < VEC; j += 4) *reinterpret_cast<f32x4*>(p + j) = f32x4{v[j], v[j + 1], v[j + 2], v[j + 3]};

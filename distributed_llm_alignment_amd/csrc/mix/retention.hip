@@ -276,7 +276,10 @@ __global__ __launch_bounds__(256) void ret_output_kernel(RetentionParams p) {
   }
 }
 
-// The recurrence, token by token. grid (H, B), NT threads; a row of the state (one v) belongs to a
+// The recurrence, token by token. grid (H, B, vsplit), NT threads; vsplit > 1 (decode of few rows): each
+// workgroup owns a range of the value rows and publishes its outputs with write-through stores; the
+// last to arrive at the (sequence, head) counter re-arms it, acquires once and does the norm and
+// gate. Nobody waits for anybody. a row of the state (one v) belongs to a
 // group of `lpr` lanes, each lane to VEC-element pieces of it.
 constexpr int kRecThreads = 512;
 template <typename T, int VEC>
@@ -294,6 +297,7 @@ __global__ __launch_bounds__(kRecThreads) void ret_recurrent_kernel(RetentionPar
   float* S = p.state + (static_cast<int64_t>(hd.b) * p.H + hd.h) * p.vdim * p.dim;
   const int grp = threadIdx.x / lpr, li = threadIdx.x % lpr, ngrp = kRecThreads / lpr;
   constexpr int U = 8;
+  const int per = (p.vdim + p.vsplit - 1) / p.vsplit, vlo = blockIdx.z * per, vhi = min(vlo + per, p.vdim);
   for (int t = 0; t < p.T; ++t) {
     const int64_t row = static_cast<int64_t>(hd.b) * p.T + t;
     const T* in = static_cast<const T*>(p.qkvg) + row * p.ld;
@@ -310,7 +314,7 @@ __global__ __launch_bounds__(kRecThreads) void ret_recurrent_kernel(RetentionPar
     for (int i = threadIdx.x; i < p.vdim; i += kRecThreads) vs[i] = pos < 0 ? 0.f : to_f<T>(in[2 * Hd + hd.h * p.vdim + i]);
     __syncthreads();
     const bool zero = p.fresh && t == 0;
-    for (int r0 = grp; r0 < p.vdim; r0 += ngrp * U) {
+    for (int r0 = vlo + grp; r0 < vhi; r0 += ngrp * U) {
       float acc[U];
 #pragma unroll
       for (int u = 0; u < U; ++u) acc[u] = 0.f;
@@ -321,12 +325,12 @@ __global__ __launch_bounds__(kRecThreads) void ret_recurrent_kernel(RetentionPar
           const int v = r0 + u * ngrp;
 #pragma unroll
           for (int e = 0; e < VEC; ++e) s[u][e] = 0.f;
-          if (v < p.vdim && !zero) load_vec<float, VEC>(S + static_cast<int64_t>(v) * p.dim + i, s[u]);
+          if (v < vhi && !zero) load_vec<float, VEC>(S + static_cast<int64_t>(v) * p.dim + i, s[u]);
         }
 #pragma unroll
         for (int u = 0; u < U; ++u) {
           const int v = r0 + u * ngrp;
-          if (v >= p.vdim) continue;
+          if (v >= vhi) continue;
 #pragma unroll
           for (int e = 0; e < VEC; ++e) {
             s[u][e] = dec * s[u][e] + ks[i + e] * vs[v];
@@ -339,8 +343,32 @@ __global__ __launch_bounds__(kRecThreads) void ret_recurrent_kernel(RetentionPar
       for (int u = 0; u < U; ++u) {
         for (int o = lpr >> 1; o > 0; o >>= 1) acc[u] += __shfl_xor(acc[u], o, 64);
         const int v = r0 + u * ngrp;
-        if (li == 0 && v < p.vdim) os[v] = acc[u];
+        if (li == 0 && v < vhi) {
+          if (p.vsplit > 1)
+            __hip_atomic_store(&p.osplit[(static_cast<int64_t>(hd.b) * p.H + hd.h) * p.vdim + v], acc[u], __ATOMIC_RELAXED,
+                               __HIP_MEMORY_SCOPE_AGENT);
+          else
+            os[v] = acc[u];
+        }
       }
+    }
+    if (p.vsplit > 1) {  // (T == 1)
+      __shared__ int last;
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      __syncthreads();
+      if (threadIdx.x == 0) {
+        int* cnt = p.cnt + static_cast<int64_t>(hd.b) * p.H + hd.h;
+        last = __hip_atomic_fetch_add(cnt, 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) == p.vsplit - 1;
+        if (last) {
+          __hip_atomic_store(cnt, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+          __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "agent");
+          asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        }
+      }
+      __syncthreads();
+      if (!last) return;
+      for (int v = threadIdx.x; v < p.vdim; v += kRecThreads)
+        os[v] = p.osplit[(static_cast<int64_t>(hd.b) * p.H + hd.h) * p.vdim + v];
     }
     __syncthreads();
     float ss = 0.f;
@@ -409,7 +437,7 @@ void recurrent(const RetentionParams& p, hipStream_t st) {
   int lpr = 1;
   while (lpr < 64 && lpr * (v4 ? 4 : 1) < p.dim) lpr *= 2;
   const int64_t lds = 4ll * (2 * round_up(p.dim, 4) + 2 * p.vdim);
-  const dim3 g(p.H, p.B);
+  const dim3 g(p.H, p.B, p.vsplit);
   if (v4) ret_recurrent_kernel<T, 4><<<g, kRecThreads, lds, st>>>(p, lpr);
   else ret_recurrent_kernel<T, 1><<<g, kRecThreads, lds, st>>>(p, lpr);
 }

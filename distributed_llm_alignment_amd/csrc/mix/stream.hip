@@ -41,10 +41,16 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(float* __restrict__ x, 
     if (c < H) load_vec<float, 4>(x + base + c, xv[j]);
 #pragma unroll
     for (int e = 0; e < 4; ++e) dv[j][e] = 0.f;
-    if (c < H && delta) {
+    if (c < H && delta) load_vec<T, 4>(delta + base + c, dv[j]);
+  }
+  float wv[NV][4], iv[NV][4];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) dv[j][e] = to_f<T>(delta[base + c + e]);
-    }
+  for (int j = 0; j < NV; ++j) {  // (in flight behind the sums)
+    const int c = 4 * (threadIdx.x + NT * j);
+    if (c < H && w) load_vec<T, 4>(w + c, wv[j]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) iv[j][e] = 0.f;
+    if (c < H && inject) load_vec<float, 4>(inject + base + c, iv[j]);
   }
   if (delta_w) {
     float ss = 0.f;
@@ -57,8 +63,10 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(float* __restrict__ x, 
     for (int j = 0; j < NV; ++j) {
       const int c = 4 * (threadIdx.x + NT * j);
       if (c < H) {
+        float dw[4];
+        load_vec<T, 4>(delta_w + c, dw);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) dv[j][e] *= r * to_f<T>(delta_w[c + e]);
+        for (int e = 0; e < 4; ++e) dv[j][e] *= r * dw[e];
       }
     }
   }
@@ -67,11 +75,9 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(float* __restrict__ x, 
   for (int j = 0; j < NV; ++j) {
     const int c = 4 * (threadIdx.x + NT * j);
     if (c >= H) continue;
-    float iv[4] = {0.f, 0.f, 0.f, 0.f};
-    if (inject) load_vec<float, 4>(inject + base + c, iv);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      xv[j][e] = xv[j][e] + dv[j][e] + iv[e];
+      xv[j][e] = xv[j][e] + dv[j][e] + iv[j][e];
       ss += xv[j][e] * xv[j][e];
     }
     if (delta || inject) store_vec<float, 4>(x + base + c, xv[j]);
@@ -81,11 +87,10 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(float* __restrict__ x, 
   for (int j = 0; j < NV; ++j) {
     const int c = 4 * (threadIdx.x + NT * j);
     if (c >= H) continue;
+    float yv[4];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const float v = w ? xv[j][e] * r * (offset + to_f<T>(w[c + e])) : xv[j][e];
-      y[base + c + e] = from_f<T>(v);
-    }
+    for (int e = 0; e < 4; ++e) yv[e] = w ? xv[j][e] * r * (offset + wv[j][e]) : xv[j][e];
+    store_vec<T, 4>(y + base + c, yv);
   }
 }
 
@@ -161,8 +166,14 @@ void norm_dispatch(float* x, const T* delta, const T* dw, const float* inject, c
                    float offset, int64_t rows, int H, hipStream_t st) {
   const dim3 g(static_cast<unsigned>(rows));
 #define DLA_NORM(NT, NV) stream_norm_kernel<T, NT, NV><<<g, NT, 0, st>>>(x, delta, dw, inject, w, y, eps, offset, H)
-  if (H % 4 || H > 16384) stream_norm_any_kernel<T><<<g, 256, 0, st>>>(x, delta, dw, inject, w, y, eps, offset, H);
+  const auto al = [](const void* q) { return reinterpret_cast<uintptr_t>(q) % 8 == 0; };
+  if (H % 4 || H > 16384 || !al(delta) || !al(dw) || !al(w) || !al(y)) stream_norm_any_kernel<T><<<g, 256, 0, st>>>(x, delta, dw, inject, w, y, eps, offset, H);
   else if (H <= 256) DLA_NORM(64, 1);
+  else if (rows <= 64 && H > 2048) {  // decode: short latency chain
+    if (H <= 4096) DLA_NORM(1024, 1);
+    else if (H <= 8192) DLA_NORM(1024, 2);
+    else DLA_NORM(1024, 4);
+  } else if (rows <= 64 && H > 1024) DLA_NORM(512, 1);
   else if (H <= 1024) DLA_NORM(256, 1);
   else if (H <= 2048) DLA_NORM(256, 2);
   else if (H <= 4096) DLA_NORM(256, 4);

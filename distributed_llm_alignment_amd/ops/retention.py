@@ -17,6 +17,20 @@ from .latent import _positions
 from .stream import _rms
 
 
+_COUNTERS = {}  # per device: arrival counters of the split decode (zero between launches)
+
+
+def _counters(device, n: int):
+    c = _COUNTERS.get(device)
+    if c is None or c.numel() < n:
+        if torch.cuda.is_current_stream_capturing():
+            return None  # never allocated (zeroed) inside a captured graph
+        # (an outgrown tensor stays alive: captured decode steps keep using it)
+        _COUNTERS.setdefault("old", []).append(c)
+        c = _COUNTERS[device] = torch.zeros(max(1024, n), dtype=torch.int32, device=device)
+    return c
+
+
 def _rotated(x, rot, cos, sin, pos):
     half = rot // 2
     c, s = cos[pos].unsqueeze(2), sin[pos].unsqueeze(2)
@@ -57,5 +71,5 @@ def decode(qkvg, H: int, dim: int, vdim: int, rot: int, eps: float, decay, state
     """One new token per row (column `base`, on the device in `slot`)."""
     if _ext.use_native(qkvg):
         return _ext.require("mix").retention_decode(qkvg, H, dim, vdim, rot, float(eps), decay, state, slot,
-                                                    kv_start, cos, sin)
+                                                    kv_start, cos, sin, _counters(qkvg.device, qkvg.shape[0] * H))
     return prefill(qkvg, H, dim, vdim, rot, eps, decay, state, slot, kv_start, cos, sin, base)

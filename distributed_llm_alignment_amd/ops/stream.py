@@ -81,7 +81,9 @@ def head_logits(h: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
 # (csrc/mix/stream_gemm.hip) few rows: the norm before a projection and the stream add / activation /
 # gate behind it run inside the projection's launch. DLA_STREAM_FUSED=0: library GEMMs + the kernels above.
 STREAM_FUSED = os.environ.get("DLA_STREAM_FUSED", "1") != "0"
-STREAM_FUSED_ROWS = int(os.environ.get("DLA_STREAM_FUSED_ROWS", "32"))
+# (17 .. 32 rows run too, but every workgroup re-reads all of a for its 16 columns: at 32 rows that is
+# more L2 traffic than the weights, and the library's GEMMs are ahead)
+STREAM_FUSED_ROWS = int(os.environ.get("DLA_STREAM_FUSED_ROWS", "16"))
 _STORE, _RELU2, _GATE, _STREAM = range(4)
 
 
