@@ -376,6 +376,8 @@ def generate(model: CausalLM, input_ids: torch.Tensor, attention_mask: Optional[
     if weight_dtype not in ("bf16", "fp8"):
         raise ValueError(f"weight_dtype must be 'bf16' or 'fp8', got {weight_dtype!r}")
     f8 = weight_dtype == "fp8" or ops.decode.fp8_enabled()
+    if f8 and model.cfg.layer_specs is not None:
+        raise ValueError(f"{model.cfg.arch}: no fp8 weight path")
     with ops.decode.fp8_weights(f8), ops.fp8_inference_scope(model, f8 and PREFILL_FP8):
         return _generate(model, input_ids, attention_mask, max_new_tokens, do_sample, temperature, top_p,
                          top_k, eos_token_id, pad_token_id, generator, return_mask, use_graph, seed)

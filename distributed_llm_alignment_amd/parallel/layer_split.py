@@ -62,6 +62,8 @@ def dispatch_layers(model, devices: Sequence[Union[str, torch.device]]):
     devs = [torch.device(d) for d in devices]
     if getattr(lm, "tp_size", 1) > 1 or getattr(lm, "_dla_fsdp", None) is not None:
         raise ValueError("layer split is a single-process mode; it does not combine with TP / FSDP")
+    if lm.cfg.layer_specs is not None:
+        raise NotImplementedError(f"{lm.cfg.arch}: per-layer designs run on one device")
     first = devs[0]
     extra = sum(p.numel() * p.element_size() for n, p in lm.named_parameters() if not n.startswith("layers."))
     plan = plan_layer_split([_layer_bytes(l) for l in lm.layers], len(devs), extra)

@@ -149,6 +149,8 @@ def apply_sequence_parallel(model, group, force: bool = False) -> Optional[Seque
     base = getattr(model, "backbone", model)
     sp = SequenceParallel(group)
     cfg = base.cfg
+    if cfg.layer_specs is not None:
+        raise NotImplementedError(f"{cfg.arch}: per-layer designs have no sequence-parallel form")
     if cfg.num_heads % sp.size or cfg.num_kv_heads % sp.size:
         raise ValueError(f"sp={sp.size} must divide num_heads={cfg.num_heads} and "
                          f"num_kv_heads={cfg.num_kv_heads}")

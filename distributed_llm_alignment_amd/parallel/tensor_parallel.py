@@ -605,6 +605,8 @@ def apply_tensor_parallel(model, group, tp_rank: Optional[int] = None, tp_size: 
     r = coll.rank(group) if tp_rank is None else tp_rank
     if tp == 1 and not (force and group is not None):
         return model
+    if cfg.layer_specs is not None:
+        raise NotImplementedError(f"{cfg.arch}: per-layer designs have no tensor-parallel form")
     if cfg.is_moe:
         raise NotImplementedError("MoE layers use expert parallelism (parallel.expert), not TP")
     if cfg.num_heads % tp or cfg.num_kv_heads % tp or cfg.intermediate_size % tp:
