@@ -152,6 +152,12 @@ __device__ __forceinline__ void load_rotated(const T* p, int i0, int rot, const 
   }
 }
 
+// 0.5 z (1 + tanh(sqrt(2 / pi) (z + 0.044715 z^3))), the tanh as 1 - 2 / (1 + e^(2u))
+__device__ __forceinline__ float gelu_tanh(float z) {
+  const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
+  return z * (1.f - 1.f / (1.f + __expf(2.f * u)));
+}
+
 __host__ __device__ constexpr int round_up(int x, int m) { return (x + m - 1) / m * m; }
 
 }  // namespace dla

@@ -13,8 +13,19 @@ __global__ __launch_bounds__(256) void embed_stream_kernel(const int64_t* __rest
   const int64_t id = ids[row];
   const bool ok = id >= 0 && id < V;
   if (!ok && threadIdx.x == 0) bad[0] = 1;
-  for (int c = threadIdx.x; c < H; c += blockDim.x)
-    out[row * H + c] = ok ? to_f<T>(table[id * H + c]) * scale : 0.f;
+  const T* src = table + (ok ? id : 0) * H;
+  const float f = ok ? scale : 0.f;
+  if (H % 4 == 0) {
+    for (int c = 4 * threadIdx.x; c < H; c += 4 * blockDim.x) {
+      float v[4];
+      load_vec<T, 4>(src + c, v);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = ok ? v[e] * f : 0.f;
+      store_vec<float, 4>(out + row * H + c, v);
+    }
+  } else {
+    for (int c = threadIdx.x; c < H; c += blockDim.x) out[row * H + c] = ok ? to_f<T>(src[c]) * f : 0.f;
+  }
 }
 
 template <int NT>
@@ -126,19 +137,22 @@ __global__ __launch_bounds__(256) void stream_norm_any_kernel(float* __restrict_
   }
 }
 
-__device__ __forceinline__ float gelu_tanh(float z) {
-  return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
-}
-
-template <typename T>
+// one wave per row
+template <typename T, int VEC>
 __global__ __launch_bounds__(256) void side_gate_kernel(const T* __restrict__ z, const int64_t* __restrict__ ids,
                                                         const T* __restrict__ table, int64_t ldt, int64_t off,
-                                                        T* __restrict__ out, int64_t n, int dim, int64_t V) {
-  for (int64_t i = blockIdx.x * 256ll + threadIdx.x; i < n; i += gridDim.x * 256ll) {
-    const int64_t row = i / dim;
-    const int64_t id = ids[row];
-    const float e = id >= 0 && id < V ? to_f<T>(table[id * ldt + off + (i - row * dim)]) : 0.f;
-    out[i] = from_f<T>(gelu_tanh(to_f<T>(z[i])) * e);
+                                                        T* __restrict__ out, int64_t rows, int dim, int64_t V) {
+  const int64_t row = blockIdx.x * 4ll + (threadIdx.x >> 6);
+  if (row >= rows) return;
+  const int64_t id = ids[row];
+  const bool ok = id >= 0 && id < V;
+  for (int c = (threadIdx.x & 63) * VEC; c < dim; c += 64 * VEC) {
+    float v[VEC], e[VEC];
+    load_vec<T, VEC>(z + row * dim + c, v);
+    load_vec<T, VEC>(table + (ok ? id : 0) * ldt + off + c, e);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] = ok ? gelu_tanh(v[j]) * e[j] : 0.f;
+    store_vec<T, VEC>(out + row * dim + c, v);
   }
 }
 
@@ -205,16 +219,20 @@ void launch_stream_norm(bool bf16, float* x, const void* delta, const void* dw, 
 
 void launch_side_gate(bool bf16, const void* z, const int64_t* ids, const void* table, int64_t ldt, int64_t off,
                       void* out, int64_t rows, int dim, int64_t V, hipStream_t st) {
-  const int64_t n = rows * dim;
-  if (n == 0) return;
-  if (bf16)
-    side_gate_kernel<bf16_t><<<grid_for(n), 256, 0, st>>>(static_cast<const bf16_t*>(z), ids,
-                                                          static_cast<const bf16_t*>(table), ldt, off,
-                                                          static_cast<bf16_t*>(out), n, dim, V);
-  else
-    side_gate_kernel<float><<<grid_for(n), 256, 0, st>>>(static_cast<const float*>(z), ids,
-                                                         static_cast<const float*>(table), ldt, off,
-                                                         static_cast<float*>(out), n, dim, V);
+  if (rows == 0) return;
+  const dim3 g(static_cast<unsigned>((rows + 3) / 4));
+  const bool vec = dim % 4 == 0 && ldt % 4 == 0 && off % 4 == 0 &&
+                   (reinterpret_cast<uintptr_t>(z) | reinterpret_cast<uintptr_t>(table) | reinterpret_cast<uintptr_t>(out)) % 16 == 0;
+#define DLA_GATE(T, V4) \
+  side_gate_kernel<T, V4><<<g, 256, 0, st>>>(static_cast<const T*>(z), ids, static_cast<const T*>(table), ldt, off, static_cast<T*>(out), rows, dim, V)
+  if (bf16) {
+    if (vec) DLA_GATE(bf16_t, 4);
+    else DLA_GATE(bf16_t, 1);
+  } else {
+    if (vec) DLA_GATE(float, 4);
+    else DLA_GATE(float, 1);
+  }
+#undef DLA_GATE
 }
 
 void launch_relu2(bool bf16, const void* u, void* y, int64_t n, hipStream_t st) {

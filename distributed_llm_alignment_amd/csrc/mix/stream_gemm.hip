@@ -95,7 +95,7 @@ __global__ __launch_bounds__(64 * kWaves) void stream_gemm_kernel(StreamGemmPara
     if (ok) {
       const int64_t id = p.ids[m];
       const float e = id >= 0 && id < p.vocab ? bf2f(p.table[id * p.ldt + p.off + n]) : 0.f;
-      v = 0.5f * v * (1.f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v))) * e;
+      v = gelu_tanh(v) * e;
     }
   }
   if constexpr (EPI == kStream) {
