@@ -25,8 +25,8 @@ def _counters(device, n: int):
     if c is None or c.numel() < n:
         if torch.cuda.is_current_stream_capturing():
             return None  # never allocated (zeroed) inside a captured graph
-        # (an outgrown tensor stays alive: captured decode steps keep using it)
-        _COUNTERS.setdefault("old", []).append(c)
+        if c is not None:  # an outgrown tensor stays alive: captured decode steps keep using it
+            _COUNTERS.setdefault("outgrown", []).append(c)
         c = _COUNTERS[device] = torch.zeros(max(1024, n), dtype=torch.int32, device=device)
     return c
 

@@ -95,15 +95,15 @@ def init_distributed(backend: Optional[str] = None, timeout_s: int = 1800,
 # a rocprofv3 trace of the ZeRO-1 bench on a forced one-rank group showed RCCL's stream on the SAME
 # hardware queue as torch's compute stream, its bucket kernels 0 % concurrent with the backward
 # (profiles/r5_force_pg_streams.md). A high-priority stream gets its own (priority) queue, so the
-# gradient collectives really run beside the backward GEMMs. DLA_RCCL_HIGH_PRIORITY=0 keeps torch's
-# default (normal-priority pool stream).
+# gradient collectives really run beside the backward GEMMs. Off by default: work on streams of
+# different priorities in one process has hung for good on this hardware pool, so every stream keeps
+# the default priority unless DLA_RCCL_HIGH_PRIORITY=1 asks otherwise.
 # The priority queue is not free: with the one-rank group's collectives in place (no RCCL kernels
 # at all), the RLHF update ran 0.405 s with it vs 0.353 s without (= the no-group run, 0.354 s),
 # and the 70B TP-8 rank step 2132 vs 2034 ms: its pending stream waits alone slow the
 # bandwidth-bound kernels of the compute queue 2-3x (profiles/r6_rlhf_forced.md). So a ONE-rank
-# group, which has nothing to overlap, keeps the normal-priority stream; groups of >= 2 ranks
-# take the high-priority one for the overlap.
-RCCL_HIGH_PRIORITY = os.environ.get("DLA_RCCL_HIGH_PRIORITY", "1") != "0"
+# group, which has nothing to overlap, keeps the normal-priority stream in any case.
+RCCL_HIGH_PRIORITY = os.environ.get("DLA_RCCL_HIGH_PRIORITY", "0") == "1"
 
 
 def comm_pg_options(group_size: int = 2):
@@ -116,7 +116,7 @@ def comm_pg_options(group_size: int = 2):
 
 
 def new_group(ranks, **kw):
-    """dist.new_group with the framework's RCCL options (high-priority comm streams)."""
+    """dist.new_group with the framework's RCCL options."""
     if _STATE.backend == "nccl" and "pg_options" not in kw:
         opts = comm_pg_options(len(ranks))
         if opts is not None:
