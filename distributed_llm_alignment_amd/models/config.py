@@ -16,7 +16,7 @@ from typing import Any, Dict, List, Optional, Tuple
 
 @dataclass
 class ModelConfig:
-    arch: str = "llama"  # llama | mistral | mixtral | gpt2 | phi | vufilorn
+    arch: str = "llama"  # llama | mistral | mixtral | gpt2 | phi | vufilorn | zenevik
     vocab_size: int = 32000
     hidden_size: int = 4096
     num_layers: int = 32
@@ -35,7 +35,7 @@ class ModelConfig:
     num_experts_per_tok: int = 2
     router_aux_loss_coef: float = 0.0
     norm_type: str = "rms"  # rms | layer
-    activation: str = "swiglu"  # swiglu | gelu_new | relu2
+    activation: str = "swiglu"  # swiglu | geglu | gelu_new | relu2
     parallel_block: bool = False  # phi: attn and mlp both read the same normed input
     attn_bias: bool = False
     mlp_bias: bool = False
@@ -53,6 +53,8 @@ class ModelConfig:
     embed_scale: float = 1.0
     norm_offset: float = 0.0  # added to the stored norm weights (1.0: weights stored around zero)
     token_side_dim: int = 0  # per-layer token input: width of each layer's slice of side_embed
+    postln_alpha: Optional[float] = None  # norm after the sum, x <- norm(alpha x + sublayer(x)); None: norm before
+    logit_softcap: float = 0.0  # logits <- cap tanh(logits / cap)
 
     @property
     def layer_schedule(self) -> List[Tuple[int, bool]]:
@@ -92,7 +94,7 @@ class ModelConfig:
             from .layer_spec import spec_param_count
 
             H, L, V = self.hidden_size, self.num_layers, self.vocab_size
-            n = H + sum(spec_param_count(self, i) for i in range(L))
+            n = H + sum(spec_param_count(self, i) for i in range(L)) + (0 if self.tie_word_embeddings else V * H)
             return n + (V * H + V * L * self.token_side_dim if include_embedding else 0)
         H, F, L = self.hidden_size, self.intermediate_size, self.num_layers
         attn = H * (self.q_size + 2 * self.kv_size) + self.q_size * H
@@ -130,8 +132,11 @@ class ModelConfig:
     # ----------------------------------------------------------------- HF config.json interop
     @classmethod
     def from_hf(cls, hf: Dict[str, Any]) -> "ModelConfig":
-        if hf.get("architecture") == "Vufilorn":
-            return cls._from_vufilorn(hf)
+        if "architecture" in hf:
+            readers = {"Vufilorn": cls._from_vufilorn, "Zenevik": cls._from_zenevik}
+            if hf["architecture"] not in readers:
+                raise ValueError(f"unsupported architecture {hf['architecture']!r} (have {sorted(readers)})")
+            return readers[hf["architecture"]](hf)
         mt = hf.get("model_type", "llama")
         if mt in ("llama", "mistral", "mixtral", "qwen2"):
             H = hf["hidden_size"]
@@ -186,11 +191,9 @@ class ModelConfig:
         """Vufilorn config.json: `layers` lists each layer's mixer (latent attention or retention)
         and feed-forward with their own sizes; the flat head / FFN fields get the largest of them
         (reporting only, the layers read their specs)."""
-        from .layer_spec import check_spec
+        from .layer_spec import checked_specs
 
-        specs = [dict(e) for e in d["layers"]]
-        for i, e in enumerate(specs):
-            check_spec(e, i)
+        specs = checked_specs(d["layers"], ("latent_attention", "retention"))
         mix = [e["mixer"] for e in specs]
         return cls(
             arch="vufilorn", vocab_size=d["vocab"], hidden_size=d["width"], num_layers=len(specs),
@@ -214,9 +217,40 @@ class ModelConfig:
                 d[k] = getattr(self, k)
         return d
 
+    @classmethod
+    def _from_zenevik(cls, d: Dict[str, Any]) -> "ModelConfig":
+        """Zenevik config.json: `layers` lists each layer's mixer (rglru, gla or attention in chunks)
+        and optional feed-forward; norms come after the sums, and the logits are soft-capped."""
+        from .layer_spec import checked_specs
+
+        specs = checked_specs(d["layers"], ("rglru", "gla", "attention"))
+        mix = [e["mixer"] for e in specs]
+        return cls(
+            arch="zenevik", vocab_size=d["vocab"], hidden_size=d["width"], num_layers=len(specs),
+            num_heads=max(m.get("heads", 1) for m in mix),
+            num_kv_heads=max(m.get("kv_heads", m.get("heads", 1)) for m in mix),
+            head_dim=max(m.get("dim", 1) for m in mix),
+            intermediate_size=max([e["mlp"]["ff"] for e in specs if e.get("mlp")], default=0),
+            norm_eps=d["norm"]["eps"], activation="geglu", tie_word_embeddings=False,
+            max_position_embeddings=d.get("max_position_embeddings", 131072), layer_specs=specs,
+            postln_alpha=float(d["postln_alpha"]), logit_softcap=float(d["logit_softcap"]),
+            # the design names no special tokens: -1 = never sampled, generation runs to its length
+            bos_token_id=d.get("bos_token_id", -1), eos_token_id=d.get("eos_token_id", -1), name="zenevik")
+
+    def _to_zenevik(self) -> Dict[str, Any]:
+        d = {"architecture": "Zenevik", "vocab": self.vocab_size, "width": self.hidden_size,
+             "norm": {"eps": self.norm_eps}, "postln_alpha": self.postln_alpha, "logit_softcap": self.logit_softcap,
+             "layers": [dict(e) for e in self.layer_specs]}
+        for k in ("bos_token_id", "eos_token_id"):
+            if getattr(self, k) >= 0:
+                d[k] = getattr(self, k)
+        return d
+
     def to_hf(self) -> Dict[str, Any]:
         if self.arch == "vufilorn":
             return self._to_vufilorn()
+        if self.arch == "zenevik":
+            return self._to_zenevik()
         if self.arch == "gpt2":
             return {"model_type": "gpt2", "architectures": ["GPT2LMHeadModel"], "vocab_size": self.vocab_size,
                     "n_embd": self.hidden_size, "n_layer": self.num_layers, "n_head": self.num_heads,
@@ -266,6 +300,15 @@ def _vufilorn_preset(vocab, width, order, ff, latent, retention, side_dim, scale
     return ModelConfig._from_vufilorn({
         "vocab": vocab, "width": width, "embedding": {"scale": scale}, "norm": {"eps": eps}, "loop": loop,
         "token_side": {"dim": side_dim}, "layers": [lat if c == "L" else ret for c in order]}).to_dict()
+
+
+def _zenevik_preset(vocab, width, order, ff, lru, gla, attn, alpha, cap=30.0, eps=1e-6):
+    """PRESETS entry of a Zenevik model: `order` is one letter per layer, R(ecurrent), G(ated linear
+    attention) or A(ttention in chunks), all layers of a kind with the same sizes."""
+    kinds = {"R": ("rglru", lru), "G": ("gla", gla), "A": ("attention", attn)}
+    return ModelConfig._from_zenevik({
+        "vocab": vocab, "width": width, "norm": {"eps": eps}, "postln_alpha": alpha, "logit_softcap": cap,
+        "layers": [{"type": kinds[c][0], "mixer": kinds[c][1], "mlp": {"kind": "dense", "ff": ff}} for c in order]}).to_dict()
 
 
 def _decays(heads: int, lo: float = 1 / 32, hi: float = 1 / 512) -> List[float]:
@@ -348,6 +391,24 @@ PRESETS.update({
         side_dim=256, scale=64.0, loop=dict(start=4, stop=16, times=2)),
 })
 
+PRESETS.update({
+    # Zenevik (real-gated recurrence, gated linear attention, attention in chunks; norm after the sum)
+    "tiny-zenevik": _zenevik_preset(
+        320, 96, "RGAR", 160, dict(width=128, blocks=4, conv=4),
+        dict(heads=3, dim=16, vdim=24, tau=8.0, rank=16),
+        dict(heads=4, kv_heads=2, dim=24, vdim=24, scale=0.2, rot=dict(base=10000.0, dims=16), mask=dict(size=11)), 2.0),
+    "zenevik-1b": _zenevik_preset(
+        32000, 2048, "RGARGARGARGARGAR", 5632, dict(width=2560, blocks=10, conv=4),
+        dict(heads=16, dim=128, vdim=128, tau=16.0, rank=16),
+        dict(heads=16, kv_heads=4, dim=128, vdim=128, scale=128 ** -0.5, rot=dict(base=1e6, dims=64),
+             mask=dict(size=4096)), 3.0),
+    "zenevik-7b": _zenevik_preset(
+        32000, 4096, "RGARGARGARGARGARGARGARGARGARGARG", 11264, dict(width=4096, blocks=16, conv=4),
+        dict(heads=16, dim=128, vdim=256, tau=16.0, rank=16),
+        dict(heads=32, kv_heads=8, dim=128, vdim=128, scale=128 ** -0.5, rot=dict(base=1e6, dims=64),
+             mask=dict(size=4096)), 3.0),
+})
+
 # HF hub ids used by the reference configs -> presets (random init offline, identical shapes)
 HUB_ALIASES = {
     "mistralai/Mistral-7B-v0.1": "mistral-7b",
@@ -377,6 +438,23 @@ def tp_shard_config(cfg: ModelConfig, tp: int) -> ModelConfig:
     return ModelConfig.from_dict(d)
 
 
+def _with_tensor_sizes(hf: Dict[str, Any], path: Path) -> Dict[str, Any]:
+    """Fill in the sizes that a per-layer design's config.json leaves to its tensors' shapes."""
+    from .layer_spec import TENSOR_SIZES
+
+    layers = hf.get("layers") if "architecture" in hf else None
+    open_sizes = [(e["mixer"], f"l{i}.{tensor}", axis, key) for i, e in enumerate(layers or [])
+                  for key, tensor, axis in TENSOR_SIZES.get(e.get("type"), ()) if key not in e["mixer"]]
+    if open_sizes:
+        from .loader import read_state_dict
+
+        sd = read_state_dict(path)
+        for mixer, tensor, axis, key in open_sizes:
+            if tensor in sd:
+                mixer[key] = int(sd[tensor].shape[axis])
+    return hf
+
+
 def get_config(name_or_path: str, **overrides) -> ModelConfig:
     """Resolve a preset / HF directory / hub alias into a ModelConfig. `<preset>@tp<N>` gives the
     per-rank shard shapes of that preset under TP degree N (tp_shard_config)."""
@@ -392,7 +470,7 @@ def get_config(name_or_path: str, **overrides) -> ModelConfig:
         if (p / "dla_config.json").exists():
             cfg = ModelConfig.from_dict(json.loads((p / "dla_config.json").read_text()))
         elif (p / "config.json").exists():
-            cfg = ModelConfig.from_hf(json.loads((p / "config.json").read_text()))
+            cfg = ModelConfig.from_hf(_with_tensor_sizes(json.loads((p / "config.json").read_text()), p))
         else:
             raise FileNotFoundError(f"{p} has no config.json")
     else:

@@ -14,6 +14,8 @@ from typing import Callable, Dict, Iterable, List, Optional, Set, Tuple
 
 import torch
 
+from .layer_spec import decay_rank
+
 _LLAMA_LIKE = ("llama", "mistral", "mixtral")
 
 
@@ -103,6 +105,40 @@ def _layer_map(cfg, i: int) -> List[Tuple[str, str, tuple]]:
             m += [(n + "side.gate", p + "side.gate", None), (n + "side.proj", p + "side.proj", None),
                   (n + "side.norm_w", p + "side.norm", None)]
         return m
+    if cfg.arch == "zenevik":
+        spec, p = cfg.layer_specs[i], f"l{i}."
+        x = spec["mixer"]
+
+        def rows(native, tensors, suffix=""):  # tensors stacked along the first dimension of one parameter
+            out, at = [], 0
+            for t, k in tensors:
+                out.append((n + native, p + "mix." + t + suffix, (at, at + k)))
+                at += k
+            return out
+
+        m = [(n + "ln1_w", p + "norm1", None)]
+        if spec["type"] == "rglru":
+            proj, gates = [("y", x["width"]), ("x", x["width"])], [("ra", x["blocks"]), ("ri", x["blocks"])]
+            m += rows("mix.in_proj", proj) + rows("mix.in_bias", proj, ".b")
+            m += rows("mix.gates", gates) + rows("mix.gates_b", gates, ".b")
+            m += [(n + "mix.conv_w", p + "mix.conv", None), (n + "mix.conv_b", p + "mix.conv.b", None),
+                  (n + "mix.lam", p + "mix.lam", None)]
+        elif spec["type"] == "gla":
+            k, v = x["heads"] * x["dim"], x["heads"] * x["vdim"]
+            m += rows("mix.in_proj", [("q", k), ("k", k), ("v", v), ("g", v), ("a1", decay_rank(x))])
+            m += [(n + "mix.decay_proj", p + "mix.a2", None), (n + "mix.decay_b", p + "mix.a2.b", None),
+                  (n + "mix.norm_w", p + "mix.norm", None)]
+        else:
+            proj = [("q", x["heads"] * x["dim"]), ("k", x["kv_heads"] * x["dim"])]
+            m += rows("mix.in_proj", proj) + rows("mix.in_bias", proj, ".b")
+            m += [(n + "mix.q_norm_w", p + "mix.q.norm", None), (n + "mix.k_norm_w", p + "mix.k.norm", None),
+                  (n + "mix.o_bias", p + "mix.o.b", None)]
+        m.append((n + "mix.o_proj", p + "mix.o", None))
+        if spec.get("mlp"):
+            f = spec["mlp"]["ff"]
+            m += [(n + "ln2_w", p + "norm2", None), (n + "mlp.up_proj", p + "mlp.gate", (0, f)),
+                  (n + "mlp.up_proj", p + "mlp.up", (f, 2 * f)), (n + "mlp.down_proj", p + "mlp.down", None)]
+        return m
     raise ValueError(cfg.arch)
 
 
@@ -119,6 +155,8 @@ def _global_map(cfg) -> List[Tuple[str, str, tuple]]:
         m = [("embed", "embed", None), ("norm_w", "final.norm", None)]
         if cfg.token_side_dim:
             m.append(("side_embed", "side.embed", None))
+    elif cfg.arch == "zenevik":
+        m = [("embed", "embed", None), ("norm_w", "final.norm", None), ("lm_head", "head", None)]
     else:
         m = [("embed", "model.embed_tokens.weight", None), ("norm_w", "model.norm.weight", None)]
         if not cfg.tie_word_embeddings:
@@ -194,7 +232,7 @@ def to_hf_state_dict(model, base: bool = False, only: Optional[Set[str]] = None)
     for native, hf, spec in key_map(model.cfg):
         if native not in params or (only is not None and native not in only):
             continue
-        if base and hf.startswith("lm_head"):
+        if base and native.startswith("lm_head"):
             continue
         t = _slice(params[native].detach(), spec)
         if spec == "T":
@@ -269,6 +307,8 @@ def load_hf_state_dict(model, sd: Mapping, strict: bool = True, base: bool = Fal
         used_out.update(used)
     if only is not None:
         return missing, []
+    if "lm_head" not in params:  # headless backbone: a checkpoint's head is not unexpected
+        used.update(hf for native, hf, _ in key_map(model.cfg) if native == "lm_head")
     unexpected = [k for k in sd if k not in used and not k.endswith("rotary_emb.inv_freq")
                   and not k.startswith("lm_head") and ".attn.bias" not in k and ".attn.masked_bias" not in k]
     if strict and (missing or unexpected):

@@ -1,10 +1,12 @@
-"""Layers of per-layer designs (`ModelConfig.layer_specs`): latent attention and retention mixers,
-squared-ReLU / other feed-forwards, the per-layer token input, and the layer that strings them
-together on an fp32 residual stream.
+"""Layers of per-layer designs (`ModelConfig.layer_specs`): latent attention, retention, real-gated
+recurrence, gated linear attention and chunked attention mixers, feed-forwards, the per-layer token
+input, and the layers that string them together on an fp32 residual stream: norm before each
+sublayer (`StreamLayer`) or after each sum (`PostNormLayer`).
 
 A `StreamLayer` never adds its own output to the stream: it hands the last projection's output on as
 the *pending* update of a `Stream`, and the next norm kernel adds it while it reads the stream (one
-pass: add, optional norm of the update, optional embedding re-injection, norm of the sum). Mixers
+pass: add, optional norm of the update, optional embedding re-injection, norm of the sum). A
+`PostNormLayer` hands its update on in the same way, with the norm that belongs to the sum. Mixers
 keep what they need of the past in a slot of `generation.KVCache` (`new_slot`); a layer that runs
 several times per forward gets one slot per run.
 """
@@ -12,14 +14,14 @@ from __future__ import annotations
 
 import dataclasses
 import math
-from typing import List, Optional
+from typing import Dict, List, Optional
 
 import torch
 import torch.nn as nn
 
 from .. import ops
 from .config import ModelConfig
-from .layer_spec import window
+from .layer_spec import decay_rank, window
 
 
 def _param(*shape, device=None, dtype=None) -> nn.Parameter:
@@ -27,13 +29,26 @@ def _param(*shape, device=None, dtype=None) -> nn.Parameter:
 
 
 @dataclasses.dataclass
+class PostNorm:
+    """What the sum alpha x + delta + bias is normed with."""
+
+    w: torch.Tensor
+    alpha: float
+    eps: float
+    bias: Optional[torch.Tensor] = None
+
+
+@dataclasses.dataclass
 class Stream:
-    """fp32 residual stream x [B, T, H] plus the update not added yet: x + norm?(delta) + inject."""
+    """fp32 residual stream x [B, T, H] plus the update not added yet: x + norm?(delta) + inject, or with
+    `post` norm(alpha x + delta + bias)."""
 
     x: torch.Tensor
     delta: Optional[torch.Tensor] = None
     delta_w: Optional[torch.Tensor] = None  # plain RMS norm of delta with this weight before the add
     inject: Optional[torch.Tensor] = None
+    post: Optional[PostNorm] = None
+    ssq: Optional[torch.Tensor] = None  # fused decode: x is the sum before `post`, these its partial sums of squares
 
     def norm(self, w, eps: float, offset: float, dtype) -> torch.Tensor:
         """Fold the pending update into x and return the normed rows."""
@@ -43,42 +58,67 @@ class Stream:
 
     def cast(self, eps: float, dtype) -> torch.Tensor:
         """Fold the pending update into x and return x in the compute dtype."""
-        return self.norm(None, eps, 0.0, dtype)
+        if self.post is None:
+            return self.norm(None, eps, 0.0, dtype)
+        return self._post(None, dtype)
+
+    def _post(self, w2, dtype) -> torch.Tensor:
+        p = self.post
+        if self.ssq is not None:  # the sum is in x already
+            y, self.x = ops.post_norm(self.x, None, None, 1.0, p.w, w2, p.eps, dtype)
+        else:
+            y, self.x = ops.post_norm(self.x, self.delta, p.bias, p.alpha, p.w, w2, p.eps, dtype)
+        self.delta = self.post = self.ssq = None
+        return y
+
+    def last_norm(self, w, eps: float, offset: float, dtype) -> torch.Tensor:
+        """The model's last norm on the finished stream."""
+        if self.post is None:
+            return self.norm(w, eps, offset, dtype)
+        return self._post(w, dtype)
 
 
 class CacheSlot:
-    """What one mixer run keeps of the past: named tensors with the batch first. `time_dim` tensors
-    have one row per token (grown by `reserve`), the others are fixed-size state."""
+    """What one mixer run keeps of the past: named tensors with the batch first. `per_token` names the
+    tensors with one row per token and the dimension of the rows (at most `limit` of them, 0: one for
+    every token; grown by `reserve`), the others are fixed-size state. `rope`: the mixer's rotary tables."""
 
-    def __init__(self, rope, max_len: int, device, **tensors):
+    def __init__(self, max_len: int, device, rope=None, per_token: Optional[Dict[str, int]] = None, limit: int = 0,
+                 **tensors):
         self.t = tensors
-        self.rope = rope
-        self.grow(max_len, device)
+        self.rope, self.per_token, self.limit = rope, per_token or {}, limit
+        self.device = device
+        self.cos = self.sin = None
+        self.grow(max_len)
 
-    def grow(self, max_len: int, device):
+    def grow(self, max_len: int):
         # the slot keeps its own reference to the rotary tables: a captured decode step reads them
         # by address, also after a longer cache made the shared RotaryCache extend
-        self.rope.ensure(max_len)
-        self.cos, self.sin = self.rope.tables(device)
+        if self.rope is not None:
+            self.rope.ensure(max_len)
+            self.cos, self.sin = self.rope.tables(self.device)
 
     def nbytes(self) -> int:
         return sum(v.numel() * v.element_size() for v in self.t.values())
 
     def keep_rows(self, rows: torch.Tensor) -> "CacheSlot":
         out = CacheSlot.__new__(CacheSlot)
-        out.rope, out.cos, out.sin = self.rope, self.cos, self.sin
+        out.__dict__.update(self.__dict__)
         out.t = {k: v.index_select(0, rows.to(v.device)) for k, v in self.t.items()}
         return out
 
     def reserve(self, max_len: int):
-        if "latent" in self.t:
-            old = self.t["latent"]
-            new = torch.zeros((old.shape[0], max_len, old.shape[2]), dtype=old.dtype, device=old.device)
-            new[:, :old.shape[1]] = old
-            self.t["latent"] = new
-            self.grow(max_len, old.device)
-        else:
-            self.grow(max_len, self.t["state"].device)
+        n = min(max_len, self.limit) if self.limit else max_len
+        for name, dim in self.per_token.items():
+            old = self.t[name]
+            if n <= old.shape[dim]:
+                continue
+            shape = list(old.shape)
+            shape[dim] = n
+            new = torch.zeros(shape, dtype=old.dtype, device=old.device)
+            new.narrow(dim, 0, old.shape[dim]).copy_(old)
+            self.t[name] = new
+        self.grow(max_len)
 
 
 class LatentAttention(nn.Module):
@@ -103,7 +143,7 @@ class LatentAttention(nn.Module):
         self.o_proj = _param(H, self.heads * self.vdim, device=device, dtype=dtype)
 
     def new_slot(self, batch: int, max_len: int, device, dtype) -> CacheSlot:
-        return CacheSlot(self.rope, max_len, device, latent=torch.zeros(
+        return CacheSlot(max_len, device, self.rope, per_token={"latent": 1}, latent=torch.zeros(
             (batch, max_len, self.kv_rank + self.rot), device=device, dtype=dtype))
 
     def mix(self, down: torch.Tensor, cache, slot: CacheSlot, lin=ops.stream_linear) -> torch.Tensor:
@@ -160,7 +200,7 @@ class Retention(nn.Module):
         return t
 
     def new_slot(self, batch: int, max_len: int, device, dtype) -> CacheSlot:
-        return CacheSlot(self.rope, max_len, device, state=torch.zeros(
+        return CacheSlot(max_len, device, self.rope, state=torch.zeros(
             (batch, self.heads, self.vdim, self.dim), device=device, dtype=torch.float32))
 
     def mix(self, qkvg: torch.Tensor, cache, slot: CacheSlot, lin=None) -> torch.Tensor:
@@ -178,7 +218,110 @@ class Retention(nn.Module):
         return (self.in_proj, self.o_proj)
 
 
-MIXERS = {"latent_attention": LatentAttention, "retention": Retention}
+class GatedRecurrence(nn.Module):
+    """Griffin's recurrent block: a gelu branch times a real-gated linear recurrence behind a short
+    convolution; its past is one fp32 state per channel and the convolution's last inputs."""
+
+    rope_key = None
+
+    def __init__(self, cfg: ModelConfig, m: dict, device=None, dtype=None):
+        super().__init__()
+        H, W, nb = cfg.hidden_size, m["width"], m["blocks"]
+        self.width, self.taps = W, m["conv"]
+        self.in_proj = _param(2 * W, H, device=device, dtype=dtype)  # rows [y; x]
+        self.in_bias = _param(2 * W, device=device, dtype=dtype)
+        self.conv_w = _param(W, self.taps, device=device, dtype=dtype)
+        self.conv_b = _param(W, device=device, dtype=dtype)
+        self.gates = _param(2 * nb, W // nb, W // nb, device=device, dtype=dtype)  # blocks of r, then of i
+        self.gates_b = _param(2 * nb, W // nb, device=device, dtype=dtype)
+        self.lam = _param(W, device=device, dtype=dtype)
+        self.o_proj = _param(H, W, device=device, dtype=dtype)
+        self.o_bias = None
+
+    def new_slot(self, batch: int, max_len: int, device, dtype) -> CacheSlot:
+        return CacheSlot(max_len, device, state=torch.zeros((batch, self.width), device=device, dtype=torch.float32),
+                         hist=torch.zeros((batch, self.taps, self.width), device=device, dtype=dtype))
+
+    def mix(self, yx: torch.Tensor, cache, slot: CacheSlot) -> torch.Tensor:
+        run = ops.lru.decode if yx.shape[1] == 1 and cache.len > 0 else ops.lru.prefill
+        return run(yx, self.in_bias, self.conv_w, self.conv_b, self.gates, self.gates_b, self.lam, slot.t["state"],
+                   slot.t["hist"], cache.slot, cache.kv_start, base=cache.len)
+
+    def matrices(self):
+        return (self.in_proj, self.o_proj)
+
+
+class GatedLinearAttention(nn.Module):
+    """Linear attention with a decay per key channel and token; its past is one fp32 state per head."""
+
+    rope_key = None
+
+    def __init__(self, cfg: ModelConfig, m: dict, device=None, dtype=None):
+        super().__init__()
+        H = cfg.hidden_size
+        self.eps, self.tau = cfg.norm_eps, float(m["tau"])
+        self.heads, self.dim, self.vdim = m["heads"], m["dim"], m["vdim"]
+        # rows [q; k; v; g; first decay projection]
+        self.in_proj = _param(2 * self.heads * (self.dim + self.vdim) + decay_rank(m), H, device=device, dtype=dtype)
+        self.decay_proj = _param(self.heads * self.dim, decay_rank(m), device=device, dtype=dtype)
+        self.decay_b = _param(self.heads * self.dim, device=device, dtype=dtype)
+        self.norm_w = _param(self.vdim, device=device, dtype=dtype)
+        self.o_proj = _param(H, self.heads * self.vdim, device=device, dtype=dtype)
+        self.o_bias = None
+
+    def new_slot(self, batch: int, max_len: int, device, dtype) -> CacheSlot:
+        return CacheSlot(max_len, device, state=torch.zeros((batch, self.heads, self.vdim, self.dim), device=device,
+                                                            dtype=torch.float32))
+
+    def mix(self, proj: torch.Tensor, cache, slot: CacheSlot) -> torch.Tensor:
+        run = ops.gla.decode if proj.shape[1] == 1 and cache.len > 0 else ops.gla.prefill
+        return run(proj, self.decay_proj, self.decay_b, self.norm_w, self.heads, self.dim, self.vdim, self.tau, self.eps,
+                   slot.t["state"], cache.slot, cache.kv_start, base=cache.len)
+
+    def matrices(self):
+        return (self.in_proj, self.o_proj)
+
+
+class ChunkAttention(nn.Module):
+    """Grouped-query attention inside chunks of the sequence, query and key normed over their whole
+    projections, the values being the projected keys; its past is the keys and values of one chunk."""
+
+    def __init__(self, cfg: ModelConfig, m: dict, device=None, dtype=None):
+        super().__init__()
+        H, n, g, d = cfg.hidden_size, m["heads"], m["kv_heads"], m["dim"]
+        self.rope_key = (m["rot"]["dims"], float(m["rot"]["base"]))
+        self.rope = None
+        self.h = ops.chunk_attention.Heads(n, g, d, m["vdim"], m["rot"]["dims"], n * d, window(m), float(m["scale"]),
+                                           cfg.norm_eps)
+        self.in_proj = _param((n + g) * d, H, device=device, dtype=dtype)  # rows [q; k]
+        self.in_bias = _param((n + g) * d, device=device, dtype=dtype)
+        self.q_norm_w = _param(n * d, device=device, dtype=dtype)
+        self.k_norm_w = _param(g * d, device=device, dtype=dtype)
+        self.o_proj = _param(H, n * m["vdim"], device=device, dtype=dtype)
+        self.o_bias = _param(H, device=device, dtype=dtype)
+
+    def new_slot(self, batch: int, max_len: int, device, dtype) -> CacheSlot:
+        h, rows = self.h, min(max_len, self.h.chunk) if self.h.chunk else max_len
+        return CacheSlot(max_len, device, self.rope, per_token={"k": 2, "v": 2}, limit=h.chunk,
+                         k=torch.zeros((batch, h.kv_heads, rows, h.dim), device=device, dtype=dtype),
+                         v=torch.zeros((batch, h.kv_heads, rows, h.vdim), device=device, dtype=dtype))
+
+    def mix(self, qk: torch.Tensor, cache, slot: CacheSlot) -> torch.Tensor:
+        att, kc, vc = ops.chunk_attention, slot.t["k"], slot.t["v"]
+        w = (self.in_bias, self.q_norm_w, self.k_norm_w)
+        if qk.shape[1] == 1 and cache.len > 0:
+            return att.decode(qk, *w, kc, vc, self.h, cache.slot, cache.kv_start, slot.cos, slot.sin, base=cache.len)
+        q, k, v = att.prepare(qk, *w, self.h, cache.kv_start, slot.cos, slot.sin, base=cache.len)
+        o = att.prefill(q, k, v, kc, vc, self.h, cache.kv_start, base=cache.len)
+        att.store(k, v, kc, vc, self.h, cache.kv_start, base=cache.len)
+        return o
+
+    def matrices(self):
+        return (self.in_proj, self.o_proj)
+
+
+MIXERS = {"latent_attention": LatentAttention, "retention": Retention, "rglru": GatedRecurrence,
+          "gla": GatedLinearAttention, "attention": ChunkAttention}
 
 
 class TokenSide(nn.Module):
@@ -252,12 +395,44 @@ class StreamLayer(nn.Module):
         return s
 
 
-def build_layers(cfg: ModelConfig, device=None, dtype=None) -> List[StreamLayer]:
+class PostNormLayer(nn.Module):
+    """One layer with its norms after the sums: x <- norm(alpha x + mixer(x)), [x <- norm(alpha x + ff(x))]."""
+
+    def __init__(self, cfg: ModelConfig, index: int, device=None, dtype=None):
+        super().__init__()
+        from .transformer import MLP
+
+        spec = cfg.layer_specs[index]
+        self.cfg, self.index = cfg, index
+        H = cfg.hidden_size
+        self.ln1_w = _param(H, device=device, dtype=dtype)
+        self.mix = MIXERS[spec["type"]](cfg, spec["mixer"], device, dtype)
+        self.mlp = None
+        if spec.get("mlp"):
+            self.ln2_w = _param(H, device=device, dtype=dtype)
+            self.mlp = MLP(dataclasses.replace(cfg, intermediate_size=spec["mlp"]["ff"]), device, dtype)
+        self.recompute = None
+
+    def forward(self, s: Stream, ids: torch.Tensor, side_embed, cache, slot: CacheSlot) -> Stream:
+        cfg, dt = self.cfg, self.ln1_w.dtype
+        a = self.mix.mix(ops.stream_linear(s.cast(cfg.norm_eps, dt), self.mix.in_proj), cache, slot)
+        s.delta = ops.stream_linear(a, self.mix.o_proj)
+        s.post = PostNorm(self.ln1_w, cfg.postln_alpha, cfg.norm_eps, self.mix.o_bias)
+        if self.mlp is not None:
+            s.delta = self.mlp(s.cast(cfg.norm_eps, dt))
+            s.post = PostNorm(self.ln2_w, cfg.postln_alpha, cfg.norm_eps)
+        return s
+
+
+def build_layers(cfg: ModelConfig, device=None, dtype=None) -> List[nn.Module]:
     """The layers of a per-layer design; mixers with equal rotary settings share one table."""
-    layers = [StreamLayer(cfg, i, device, dtype) for i in range(cfg.num_layers)]
+    kind = StreamLayer if cfg.postln_alpha is None else PostNormLayer
+    layers = [kind(cfg, i, device, dtype) for i in range(cfg.num_layers)]
     ropes = {}
     for layer in layers:
         key = layer.mix.rope_key
+        if key is None:
+            continue
         if key not in ropes:
             ropes[key] = ops.RotaryCache(key[0], key[1], 256)
         layer.mix.rope = ropes[key]

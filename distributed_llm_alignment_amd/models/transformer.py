@@ -3,7 +3,7 @@
 One implementation, configured by `ModelConfig`, covers Llama-3 / Mistral (RMSNorm, GQA, RoPE,
 SwiGLU, optional sliding window), Mixtral (top-k routed SwiGLU experts), GPT-2 (LayerNorm,
 learned positions, GELU, tied head) and phi-2 (parallel attn+MLP block, partial rotary, biases);
-designs whose layers differ from each other (`ModelConfig.layer_specs`: Vufilorn) take their layers
+designs whose layers differ from each other (`ModelConfig.layer_specs`: Vufilorn, Zenevik) take their layers
 from models/mixers.py and run on an fp32 residual stream, with the same embedding / cache / head /
 generation around them.
 It replaces the HF modeling code the reference runs through `AutoModelForCausalLM`
@@ -145,6 +145,8 @@ class Attention(nn.Module):
 def _act(cfg: ModelConfig, u: torch.Tensor) -> torch.Tensor:
     if cfg.activation == "swiglu":
         return ops.swiglu(u)
+    if cfg.activation == "geglu":
+        return ops.geglu(u)
     return ops.relu2(u) if cfg.activation == "relu2" else ops.gelu_new(u)
 
 
@@ -153,7 +155,7 @@ class MLP(nn.Module):
         super().__init__()
         self.cfg = cfg
         H, Fd = cfg.hidden_size, cfg.intermediate_size
-        if cfg.activation == "swiglu":
+        if cfg.activation in ("swiglu", "geglu"):
             self.up_proj = _param(2 * Fd, H, device=device, dtype=dtype)  # [gate; up]
         else:
             self.up_proj = _param(Fd, H, device=device, dtype=dtype)
@@ -570,7 +572,7 @@ class CausalLM(nn.Module):
             if add:
                 s.inject = x0
             s = self.layers[i](s, input_ids, self.side_embed, cache, cache.slots[j])
-        h = s.norm(self.norm_w, cfg.norm_eps, cfg.norm_offset, self.embed.dtype)
+        h = s.last_norm(self.norm_w, cfg.norm_eps, cfg.norm_offset, self.embed.dtype)
         cache.step_done(input_ids.shape[1])
         return h
 
@@ -615,7 +617,8 @@ class CausalLM(nn.Module):
 
     def logits(self, hidden: torch.Tensor) -> torch.Tensor:
         if self.cfg.layer_specs is not None:
-            return ops.head_logits(hidden, self.head_weight)
+            lg = ops.head_logits(hidden, self.head_weight)
+            return ops.softcap(lg, self.cfg.logit_softcap) if self.cfg.logit_softcap else lg
         lg = None
         if self.lm_head_bias is None and self.vocab_parallel is None:
             lg = ops.decode.head_f8(hidden, self.head_weight)  # fp8 decode mode only
@@ -653,9 +656,9 @@ class CausalLM(nn.Module):
 
     def _masked_token_logprob(self, h: torch.Tensor, tgt: torch.Tensor) -> torch.Tensor:
         """[S, T', H] hidden + [S, T'] targets (-100 = ignore) -> [S, T'] fp32 log-probs (0 where
-        ignored); the LM-head bias models (phi-2) go through full logits."""
+        ignored); models with an LM-head bias (phi-2) or a logit soft cap go through full logits."""
         S, T, H = h.shape
-        if self.lm_head_bias is not None:
+        if self.lm_head_bias is not None or self.cfg.logit_softcap:
             lg = self.logits(h).float()
             lp = torch.log_softmax(lg, -1).gather(-1, tgt.clamp(min=0).unsqueeze(-1)).squeeze(-1)
             return torch.where(tgt >= 0, lp, torch.zeros_like(lp))
@@ -733,13 +736,14 @@ def _param_seed(seed: int, idx: int) -> int:
 
 def init_param_tensor(cfg: ModelConfig, name: str, idx: int, shape, seed: int, device, dtype) -> torch.Tensor:
     """The init value of parameter `name` (index `idx` in named_parameters order) as a fresh
-    tensor: norm weights 1, other vectors 0, matrices N(0, init_std) with the GPT-2 style
+    tensor: norm weights 1, other vectors 0 (decay parameters: slow decays), matrices N(0, init_std) with the GPT-2 style
     1/sqrt(2L) scaling on the residual-output projections."""
     device = torch.device(device)
     if len(shape) == 1:
         val = 1.0 if name.endswith(("ln1_w", "ln2_w", "norm_w")) else 0.0
         if name.endswith(("ln1_w", "ln2_w")) or name == "norm_w":
             val -= cfg.norm_offset
+        val = {"lam": -4.0, "decay_b": 2.0}.get(name.rsplit(".", 1)[-1], val)
         return torch.full(shape, val, device=device, dtype=dtype)
     std = cfg.init_std
     if name.endswith(("o_proj", "down_proj", "expert_down")):

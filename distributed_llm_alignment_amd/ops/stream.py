@@ -48,6 +48,21 @@ def stream_norm(x: torch.Tensor, delta: Optional[torch.Tensor], delta_w: Optiona
     return y.to(dtype), x
 
 
+def post_norm(x: torch.Tensor, delta: Optional[torch.Tensor], bias: Optional[torch.Tensor], alpha: float, w: torch.Tensor,
+              w2: Optional[torch.Tensor], eps: float, dtype: torch.dtype) -> Tuple[torch.Tensor, torch.Tensor]:
+    """Norm after the sum: x <- RMSNorm(alpha x + delta + bias) * w (fp32); y = x, or RMSNorm(x) * w2
+    when w2 is given (the model's last norm), in `dtype`. Returns (y, x); the GPU kernel updates x in
+    place."""
+    if _ext.use_native(x):
+        y = _ext.require("mix").post_norm(x, delta, bias, float(alpha), w, w2, float(eps), dtype == torch.bfloat16)
+        return y, x
+    s = alpha * x if delta is None else alpha * x + delta.float()
+    if bias is not None:
+        s = s + bias.float()
+    x = _rms(s, eps) * w.float()
+    return (x if w2 is None else _rms(x, eps) * w2.float()).to(dtype), x
+
+
 def side_gate(z: torch.Tensor, ids: torch.Tensor, side_embed: torch.Tensor, off: int) -> torch.Tensor:
     """gelu_tanh(z) * side_embed[ids, off : off + z.shape[-1]]."""
     if _ext.use_native(z):
@@ -63,6 +78,23 @@ def relu2(u: torch.Tensor) -> torch.Tensor:
             raise NotImplementedError("relu2 on the GPU is inference only")
         return _ext.require("mix").relu2(u)
     return torch.relu(u.float()).square().to(u.dtype)
+
+
+def geglu(u: torch.Tensor) -> torch.Tensor:
+    """u [.., 2 F] = [gate | up] -> gelu_tanh(gate) * up."""
+    if _ext.use_native(u):
+        if torch.is_grad_enabled() and u.requires_grad:
+            raise NotImplementedError("geglu on the GPU is inference only")
+        return _ext.require("mix").geglu(u)
+    gate, up = u.float().chunk(2, -1)
+    return (F.gelu(gate, approximate="tanh") * up).to(u.dtype)
+
+
+def softcap(z: torch.Tensor, cap: float) -> torch.Tensor:
+    """cap * tanh(z / cap), fp32."""
+    if _ext.use_native(z):
+        return _ext.require("mix").softcap(z, float(cap))
+    return cap * torch.tanh(z.float() / cap)
 
 
 def stream_linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
