@@ -1,5 +1,5 @@
-// torch.ops.dla ops of the mixer library (_C_mix.so): the fp32 residual stream, latent attention and
-// retention of per-layer designs. Host-side validation only; bf16 and fp32 tensors.
+// torch.ops.dla ops of the mixer library (_C_mix.so): the fp32 residual stream and the mixers of
+// per-layer designs. Host-side validation only; bf16 and fp32 tensors.
 #include <ATen/ATen.h>
 #include <torch/library.h>
 
@@ -30,6 +30,23 @@ void launch_latent_prefill_mfma(const LatentParams&, hipStream_t);
 void launch_latent_prefill_any(bool, const LatentParams&, hipStream_t);
 int latent_decode_tile(bool, const LatentParams&);
 void launch_latent_decode(bool, const LatentParams&, int, hipStream_t);
+
+void launch_post_norm(bool, float*, const void*, const void*, float, const void*, const void*, void*, float, int64_t, int,
+                      hipStream_t);
+void launch_geglu(bool, const void*, void*, int64_t, int, hipStream_t);
+void launch_softcap(bool, const void*, float*, int64_t, float, hipStream_t);
+int lru_chunk(const LruParams&);
+void launch_lru_prefill(bool, const LruParams&, hipStream_t);
+void launch_lru_decode(bool, const LruParams&, hipStream_t);
+int gla_chunks(bool, const GlaParams&);
+void launch_gla_prefill(const GlaParams&, hipStream_t);
+void launch_gla_recurrent(bool, const GlaParams&, hipStream_t);
+void launch_chunk_prepare(bool, const ChunkAttnParams&, bool, hipStream_t);
+void launch_chunk_store(bool, const ChunkAttnParams&, hipStream_t);
+bool chunk_prefill_mfma_ok(const ChunkAttnParams&);
+void launch_chunk_prefill_mfma(const ChunkAttnParams&, hipStream_t);
+void launch_chunk_prefill_any(bool, const ChunkAttnParams&, hipStream_t);
+void launch_chunk_decode(bool, const ChunkAttnParams&, hipStream_t);
 
 void launch_stream_gemm(const StreamGemmParams&, int, hipStream_t);
 
@@ -119,6 +136,52 @@ at::Tensor stream_norm(at::Tensor x, const OptT& delta, const OptT& delta_w, con
                      delta_w.has_value() ? delta_w->data_ptr() : nullptr,
                      inject.has_value() ? inject->data_ptr<float>() : nullptr, w.has_value() ? w->data_ptr() : nullptr,
                      y.data_ptr(), static_cast<float>(eps), static_cast<float>(offset), rows, static_cast<int>(H), cur_stream(x));
+  return y;
+}
+
+at::Tensor post_norm(at::Tensor x, const OptT& delta, const OptT& bias, double alpha, const at::Tensor& w, const OptT& w2,
+                     double eps, bool bf16) {
+  check_f32(x, "x");
+  TORCH_CHECK(x.dim() >= 1 && x.is_contiguous() && x.size(-1) > 0, "x contiguous [.., H]");
+  const int64_t H = x.size(-1), rows = x.numel() / H;
+  TORCH_CHECK(rows < (1ll << 31) && H < (1 << 24), "x too large");
+  auto y = at::empty(x.sizes(), x.options().dtype(bf16 ? at::kBFloat16 : at::kFloat));
+  at::Tensor d;
+  if (delta.has_value()) {
+    d = delta->contiguous();
+    like(d, y, "delta");
+    TORCH_CHECK(d.numel() == x.numel() && d.size(-1) == H, "delta like x");
+  }
+  vec_like(w, y, H, "w");
+  if (bias.has_value()) vec_like(*bias, y, H, "bias");
+  if (w2.has_value()) vec_like(*w2, y, H, "w2");
+  check_aligned16(x, "x");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(x.device());
+  launch_post_norm(bf16, x.data_ptr<float>(), d.defined() ? d.data_ptr() : nullptr, bias.has_value() ? bias->data_ptr() : nullptr,
+                   static_cast<float>(alpha), w.data_ptr(), w2.has_value() ? w2->data_ptr() : nullptr, y.data_ptr(),
+                   static_cast<float>(eps), rows, static_cast<int>(H), cur_stream(x));
+  return y;
+}
+
+at::Tensor geglu(const at::Tensor& u_) {
+  const bool bf = elem(u_, "u");
+  const at::Tensor u = u_.contiguous();
+  TORCH_CHECK(u.dim() >= 1 && u.size(-1) > 0 && u.size(-1) % 2 == 0 && u.size(-1) < (1ll << 31), "geglu: u [.., 2 F]");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(u.device());
+  auto shape = u.sizes().vec();
+  shape.back() /= 2;
+  auto y = at::empty(shape, u.options());
+  launch_geglu(bf, u.data_ptr(), y.data_ptr(), y.numel() / shape.back(), static_cast<int>(shape.back()), cur_stream(u));
+  return y;
+}
+
+at::Tensor softcap(const at::Tensor& z_, double cap) {
+  const bool bf = elem(z_, "z");
+  TORCH_CHECK(cap > 0, "softcap: cap > 0");
+  const at::Tensor z = z_.contiguous();
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(z.device());
+  auto y = at::empty(z.sizes(), z.options().dtype(at::kFloat));
+  launch_softcap(bf, z.data_ptr(), y.data_ptr<float>(), z.numel(), static_cast<float>(cap), cur_stream(z));
   return y;
 }
 
@@ -296,6 +359,329 @@ at::Tensor retention_decode(const at::Tensor& qkvg, int64_t H, int64_t dim, int6
   return y;
 }
 
+// ---- gated linear recurrence ----
+LruParams lru_params(const at::Tensor& yx, const at::Tensor& bias, const at::Tensor& conv_w, const at::Tensor& conv_b,
+                     const at::Tensor& gates, const at::Tensor& gates_b, const at::Tensor& lam, double c,
+                     const at::Tensor& state, const at::Tensor& hist, const OptT& kv_start) {
+  elem(yx, "yx");
+  like(conv_w, yx, "conv_w");
+  TORCH_CHECK(conv_w.dim() == 2 && conv_w.is_contiguous() && conv_w.size(0) > 0 && conv_w.size(1) > 0 && conv_w.size(1) < 1024,
+              "conv_w [W, taps]");
+  const int64_t W = conv_w.size(0), taps = conv_w.size(1);
+  TORCH_CHECK(yx.dim() == 3 && yx.is_contiguous() && yx.size(2) == 2 * W, "yx [B, T, 2 W] contiguous");
+  const int64_t B = yx.size(0), T = yx.size(1);
+  TORCH_CHECK(B > 0 && T > 0 && B < 65536 && T < (1ll << 30) && W < (1ll << 24), "lru: shape");
+  vec_like(bias, yx, 2 * W, "bias");
+  vec_like(conv_b, yx, W, "conv_b");
+  vec_like(lam, yx, W, "lam");
+  like(gates, yx, "gates");
+  like(gates_b, yx, "gates_b");
+  TORCH_CHECK(gates.dim() == 3 && gates.is_contiguous() && gates.size(0) > 0 && gates.size(0) % 2 == 0 &&
+                  gates.size(1) == gates.size(2) && gates.size(0) / 2 * gates.size(1) == W,
+              "gates [2 blocks, n, n], blocks * n = W");
+  TORCH_CHECK(gates_b.is_contiguous() && gates_b.sizes() == at::IntArrayRef({gates.size(0), gates.size(1)}), "gates_b [2 blocks, n]");
+  check_f32(state, "state");
+  same_device(yx, state);
+  TORCH_CHECK(state.is_contiguous() && state.sizes() == at::IntArrayRef({B, W}), "state fp32 [B, W]");
+  like(hist, yx, "hist");
+  TORCH_CHECK(hist.is_contiguous() && hist.sizes() == at::IntArrayRef({B, taps, W}), "hist [B, taps, W]");
+  LruParams p{};
+  p.yx = yx.data_ptr();
+  p.bias = bias.data_ptr();
+  p.conv_w = conv_w.data_ptr();
+  p.conv_b = conv_b.data_ptr();
+  p.gates = gates.data_ptr();
+  p.gates_b = gates_b.data_ptr();
+  p.lam = lam.data_ptr();
+  p.state = state.data_ptr<float>();
+  p.hist = hist.data_ptr();
+  p.kv_start = starts(kv_start, yx, B);
+  p.c = static_cast<float>(c);
+  p.B = static_cast<int>(B);
+  p.T = static_cast<int>(T);
+  p.W = static_cast<int>(W);
+  p.taps = static_cast<int>(taps);
+  p.nb = static_cast<int>(gates.size(0) / 2);
+  p.n = static_cast<int>(gates.size(1));
+  TORCH_CHECK(static_cast<int64_t>(p.nb) * ((p.n + 127) / 128) < 65536, "lru: too many gate blocks");
+  return p;
+}
+
+at::Tensor lru_prefill(const at::Tensor& yx, const at::Tensor& bias, const at::Tensor& conv_w, const at::Tensor& conv_b,
+                       const at::Tensor& gates, const at::Tensor& gates_b, const at::Tensor& lam, double c, at::Tensor state,
+                       at::Tensor hist, const OptT& kv_start, int64_t base) {
+  LruParams p = lru_params(yx, bias, conv_w, conv_b, gates, gates_b, lam, c, state, hist, kv_start);
+  TORCH_CHECK(base >= 0 && base < (1ll << 40) && (p.T + 3) / 4 < 65536, "lru_prefill: portion too long");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(yx.device());
+  auto out = at::empty({p.B, p.T, p.W}, yx.options());
+  p.out = out.data_ptr();
+  p.base = base;
+  p.chunk = lru_chunk(p);
+  p.nc = (p.T + p.chunk - 1) / p.chunk;
+  auto cum = at::empty({p.B, p.T, p.W}, state.options()), loc = at::empty({p.B, p.T, p.W}, state.options());
+  auto start = at::empty({p.B, p.nc, p.W}, state.options());
+  p.cum = cum.data_ptr<float>();
+  p.loc = loc.data_ptr<float>();
+  p.start = start.data_ptr<float>();
+  launch_lru_prefill(yx.scalar_type() == at::kBFloat16, p, cur_stream(yx));
+  return out;
+}
+
+at::Tensor lru_decode(const at::Tensor& yx, const at::Tensor& bias, const at::Tensor& conv_w, const at::Tensor& conv_b,
+                      const at::Tensor& gates, const at::Tensor& gates_b, const at::Tensor& lam, double c, at::Tensor state,
+                      at::Tensor hist, const at::Tensor& slot, const OptT& kv_start) {
+  LruParams p = lru_params(yx, bias, conv_w, conv_b, gates, gates_b, lam, c, state, hist, kv_start);
+  TORCH_CHECK(p.T == 1, "lru_decode: one token per row");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(yx.device());
+  auto out = at::empty({p.B, 1, p.W}, yx.options());
+  p.out = out.data_ptr();
+  p.slot = slot_ptr(slot, yx);
+  launch_lru_decode(yx.scalar_type() == at::kBFloat16, p, cur_stream(yx));
+  return out;
+}
+
+// ---- gated linear attention ----
+GlaParams gla_params(const at::Tensor& proj, const at::Tensor& a2, const at::Tensor& a2_b, const at::Tensor& norm_w, int64_t H,
+                     int64_t dim, int64_t vdim, double tau, double eps, const at::Tensor& state) {
+  elem(proj, "proj");
+  like(a2, proj, "a2");
+  TORCH_CHECK(a2.dim() == 2 && a2.is_contiguous() && H > 0 && dim > 0 && vdim > 0 && a2.size(0) == H * dim && a2.size(1) > 0 && tau > 0,
+              "a2 [H dim, rank]");
+  TORCH_CHECK(proj.dim() == 3 && proj.is_contiguous() && proj.size(2) == 2 * H * (dim + vdim) + a2.size(1),
+              "proj [B, T, 2 H (dim + vdim) + rank] contiguous");
+  const int64_t B = proj.size(0), T = proj.size(1);
+  TORCH_CHECK(B > 0 && T > 0 && B < 65536 && H < 65536 && T < (1ll << 30) && H * dim < (1ll << 21), "gla: shape");
+  vec_like(a2_b, proj, H * dim, "a2_b");
+  vec_like(norm_w, proj, vdim, "norm_w");
+  check_f32(state, "state");
+  same_device(proj, state);
+  TORCH_CHECK(state.is_contiguous() && state.sizes() == at::IntArrayRef({B, H, vdim, dim}), "state fp32 [B, H, vdim, dim]");
+  check_aligned16(state, "state");
+  GlaParams p{};
+  p.proj = proj.data_ptr();
+  p.ld = proj.size(2);
+  p.a2 = a2.data_ptr();
+  p.a2_b = a2_b.data_ptr();
+  p.norm_w = norm_w.data_ptr();
+  p.state = state.data_ptr<float>();
+  p.B = static_cast<int>(B);
+  p.T = static_cast<int>(T);
+  p.H = static_cast<int>(H);
+  p.dim = static_cast<int>(dim);
+  p.vdim = static_cast<int>(vdim);
+  p.rank = static_cast<int>(a2.size(1));
+  p.eps = static_cast<float>(eps);
+  p.inv_tau = static_cast<float>(1.0 / tau);
+  p.qscale = 1.f / std::sqrt(static_cast<float>(dim));
+  p.vsplit = 1;
+  TORCH_CHECK(gla_recurrent_lds(p) <= 60 * 1024, "gla: head sizes too large");
+  return p;
+}
+
+at::Tensor gla_prefill(const at::Tensor& proj, const at::Tensor& a2, const at::Tensor& a2_b, const at::Tensor& norm_w, int64_t H,
+                       int64_t dim, int64_t vdim, double tau, double eps, at::Tensor state, const OptT& kv_start, int64_t base) {
+  GlaParams p = gla_params(proj, a2, a2_b, norm_w, H, dim, vdim, tau, eps, state);
+  TORCH_CHECK(base >= 0 && base < (1ll << 40), "gla_prefill: base");
+  const bool bf = proj.scalar_type() == at::kBFloat16;
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(proj.device());
+  auto y = at::empty({p.B, p.T, H * vdim}, proj.options());
+  p.y = y.data_ptr();
+  p.base = base;
+  p.fresh = base == 0;
+  p.kv_start = starts(kv_start, proj, p.B);
+  p.nc = gla_chunks(bf, p);
+  if (p.nc == 0) {
+    launch_gla_recurrent(bf, p, cur_stream(proj));
+    return y;
+  }
+  auto work = at::empty({p.B, H, p.nc, vdim, dim}, state.options());
+  auto cum = at::empty({p.B, p.T, H * dim}, state.options()), total = at::empty({p.B, p.nc, H * dim}, state.options());
+  p.work = work.data_ptr<float>();
+  p.cum = cum.data_ptr<float>();
+  p.total = total.data_ptr<float>();
+  launch_gla_prefill(p, cur_stream(proj));
+  return y;
+}
+
+at::Tensor gla_decode(const at::Tensor& proj, const at::Tensor& a2, const at::Tensor& a2_b, const at::Tensor& norm_w, int64_t H,
+                      int64_t dim, int64_t vdim, double tau, double eps, at::Tensor state, const OptT& cnt) {
+  GlaParams p = gla_params(proj, a2, a2_b, norm_w, H, dim, vdim, tau, eps, state);
+  TORCH_CHECK(p.T == 1, "gla_decode: one token per row");
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(proj.device());
+  auto y = at::empty({p.B, 1, H * vdim}, proj.options());
+  p.y = y.data_ptr();
+  // few (sequence, head) pairs with a large state (>= 128 KB): several workgroups share the value rows
+  at::Tensor part;
+  if (cnt.has_value() && dim * vdim >= 32 * 1024) {
+    check_i32(*cnt, "cnt");
+    TORCH_CHECK(cnt->is_contiguous() && cnt->numel() >= p.B * H && cnt->device() == proj.device(), "cnt int32, >= B H");
+    int64_t vs = std::min<int64_t>(512 / std::max<int64_t>(1, p.B * H), vdim / 32);
+    vs = std::min<int64_t>(vs, 8);
+    if (vs > 1) {
+      part = at::empty({p.B, H, vdim}, state.options());
+      p.osplit = part.data_ptr<float>();
+      p.cnt = cnt->data_ptr<int>();
+      p.vsplit = static_cast<int>(vs);
+    }
+  }
+  launch_gla_recurrent(proj.scalar_type() == at::kBFloat16, p, cur_stream(proj));
+  return y;
+}
+
+// ---- attention inside chunks ----
+constexpr int64_t kNoChunks = 1 << 30;
+
+ChunkAttnParams chunk_sizes(int64_t B, int64_t T, int64_t H, int64_t G, int64_t dim, int64_t vdim, int64_t chunk, double scale) {
+  TORCH_CHECK(B > 0 && T > 0 && H > 0 && G > 0 && H % G == 0 && dim > 0 && vdim > 0 && chunk >= 0 && chunk <= kNoChunks && B < 65536 &&
+                  H < 65536 && T < (1ll << 30) && B * T < (1ll << 31) && dim + vdim <= 4096,
+              "chunk attention: shape");
+  ChunkAttnParams p{};
+  p.B = static_cast<int>(B);
+  p.T = static_cast<int>(T);
+  p.H = static_cast<int>(H);
+  p.G = static_cast<int>(G);
+  p.dim = static_cast<int>(dim);
+  p.vdim = static_cast<int>(vdim);
+  p.chunk = static_cast<int>(chunk > 0 ? chunk : kNoChunks);
+  p.scale = static_cast<float>(scale);
+  return p;
+}
+
+void chunk_row(ChunkAttnParams& p, const at::Tensor& row, const at::Tensor& bias, const at::Tensor& q_w, const at::Tensor& k_w,
+               int64_t rot, int64_t v_off, double eps, const at::Tensor& cos_t, const at::Tensor& sin_t) {
+  const int64_t nq = static_cast<int64_t>(p.H) * p.dim, nk = static_cast<int64_t>(p.G) * p.dim, nv = static_cast<int64_t>(p.G) * p.vdim;
+  TORCH_CHECK(row.is_contiguous() && row.size(2) >= nq + nk && v_off >= 0 && v_off + nv <= row.size(2) && rot >= 0 && rot <= p.dim,
+              "row [B, T, >= (H + G) dim] with the values at v_off");
+  vec_like(bias, row, row.size(2), "bias");
+  vec_like(q_w, row, nq, "q_w");
+  vec_like(k_w, row, nk, "k_w");
+  p.row = row.data_ptr();
+  p.ld = row.size(2);
+  p.bias = bias.data_ptr();
+  p.q_w = q_w.data_ptr();
+  p.k_w = k_w.data_ptr();
+  p.eps = static_cast<float>(eps);
+  p.rot = static_cast<int>(rot);
+  p.v_off = static_cast<int>(v_off);
+  p.npos = static_cast<int>(tables(cos_t, sin_t, rot, row));
+  p.cos_t = cos_t.data_ptr<float>();
+  p.sin_t = sin_t.data_ptr<float>();
+}
+
+void chunk_cache(ChunkAttnParams& p, const at::Tensor& kc, const at::Tensor& vc, const at::Tensor& ref) {
+  like(kc, ref, "kc");
+  like(vc, ref, "vc");
+  TORCH_CHECK(kc.dim() == 4 && kc.is_contiguous() && vc.is_contiguous() && kc.size(2) > 0 && kc.size(2) < (1ll << 30) &&
+                  kc.sizes() == at::IntArrayRef({p.B, p.G, kc.size(2), p.dim}) &&
+                  vc.sizes() == at::IntArrayRef({p.B, p.G, kc.size(2), p.vdim}),
+              "cache [B, G, rows, dim] / [B, G, rows, vdim] contiguous");
+  p.rows = static_cast<int>(kc.size(2));
+  p.kc = kc.data_ptr();
+  p.vc = vc.data_ptr();
+}
+
+std::tuple<at::Tensor, at::Tensor, at::Tensor> chunk_prepare(const at::Tensor& row, const at::Tensor& bias, const at::Tensor& q_w,
+                                                             const at::Tensor& k_w, int64_t H, int64_t G, int64_t dim,
+                                                             int64_t vdim, int64_t rot, int64_t v_off, double eps,
+                                                             const OptT& kv_start, const at::Tensor& cos_t,
+                                                             const at::Tensor& sin_t, int64_t base) {
+  const bool bf = elem(row, "row");
+  TORCH_CHECK(row.dim() == 3, "row [B, T, columns]");
+  ChunkAttnParams p = chunk_sizes(row.size(0), row.size(1), H, G, dim, vdim, 0, 1.0);
+  chunk_row(p, row, bias, q_w, k_w, rot, v_off, eps, cos_t, sin_t);
+  TORCH_CHECK(base >= 0 && (rot == 0 || base + p.T <= p.npos), "positions exceed the rotary table");
+  p.kv_start = starts(kv_start, row, p.B);
+  p.base = base;
+  p.rows = 1;
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(row.device());
+  auto q = at::empty({p.B, p.T, H, dim}, row.options()), k = at::empty({p.B, p.T, G, dim}, row.options());
+  auto v = at::empty({p.B, p.T, G, vdim}, row.options());
+  p.q = q.data_ptr();
+  p.k = k.data_ptr();
+  p.v = v.data_ptr();
+  launch_chunk_prepare(bf, p, false, cur_stream(row));
+  return {q, k, v};
+}
+
+void chunk_kv(ChunkAttnParams& p, const at::Tensor& k, const at::Tensor& v) {
+  p.k = k.data_ptr();
+  p.v = v.data_ptr();
+}
+
+at::Tensor chunk_prefill(const at::Tensor& q, const at::Tensor& k, const at::Tensor& v, const at::Tensor& kc, const at::Tensor& vc,
+                         int64_t chunk, double scale, const OptT& kv_start, int64_t base) {
+  const bool bf = elem(q, "q");
+  like(k, q, "k");
+  like(v, q, "v");
+  TORCH_CHECK(q.dim() == 4 && k.dim() == 4 && v.dim() == 4 && q.is_contiguous() && k.is_contiguous() && v.is_contiguous() &&
+                  k.sizes() == at::IntArrayRef({q.size(0), q.size(1), k.size(2), q.size(3)}) &&
+                  v.sizes() == at::IntArrayRef({q.size(0), q.size(1), k.size(2), v.size(3)}),
+              "q [B, T, H, dim], k [B, T, G, dim], v [B, T, G, vdim] contiguous");
+  ChunkAttnParams p = chunk_sizes(q.size(0), q.size(1), q.size(2), k.size(2), q.size(3), v.size(3), chunk, scale);
+  chunk_cache(p, kc, vc, q);
+  // every earlier position of the portion's first chunk has a row
+  TORCH_CHECK(base >= 0 && base + p.T < kNoChunks && std::min<int64_t>(base, p.chunk) <= p.rows, "chunk_prefill: cache rows");
+  chunk_kv(p, k, v);
+  p.q = q.data_ptr();
+  p.kv_start = starts(kv_start, q, p.B);
+  p.base = base;
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(q.device());
+  auto o = at::empty({p.B, p.T, static_cast<int64_t>(p.H) * p.vdim}, q.options());
+  p.o = o.data_ptr();
+  if (bf && chunk_prefill_mfma_ok(p)) launch_chunk_prefill_mfma(p, cur_stream(q));
+  else launch_chunk_prefill_any(bf, p, cur_stream(q));
+  return o;
+}
+
+void chunk_store(const at::Tensor& k, const at::Tensor& v, at::Tensor kc, at::Tensor vc, int64_t chunk, const OptT& kv_start,
+                 int64_t base) {
+  const bool bf = elem(k, "k");
+  like(v, k, "v");
+  TORCH_CHECK(k.dim() == 4 && v.dim() == 4 && k.is_contiguous() && v.is_contiguous() &&
+                  v.sizes() == at::IntArrayRef({k.size(0), k.size(1), k.size(2), v.size(3)}),
+              "k [B, T, G, dim], v [B, T, G, vdim] contiguous");
+  ChunkAttnParams p = chunk_sizes(k.size(0), k.size(1), k.size(2), k.size(2), k.size(3), v.size(3), chunk, 1.0);
+  chunk_cache(p, kc, vc, k);
+  TORCH_CHECK(base >= 0 && std::min<int64_t>(base + p.T, p.chunk) <= p.rows, "chunk_store: cache rows");
+  chunk_kv(p, k, v);
+  p.kv_start = starts(kv_start, k, p.B);
+  p.base = base;
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(k.device());
+  launch_chunk_store(bf, p, cur_stream(k));
+}
+
+at::Tensor chunk_decode(const at::Tensor& row, const at::Tensor& bias, const at::Tensor& q_w, const at::Tensor& k_w, int64_t H,
+                        int64_t G, int64_t dim, int64_t vdim, int64_t rot, int64_t v_off, double eps, at::Tensor kc,
+                        at::Tensor vc, int64_t chunk, double scale, const at::Tensor& slot, const OptT& kv_start,
+                        const at::Tensor& cos_t, const at::Tensor& sin_t) {
+  const bool bf = elem(row, "row");
+  TORCH_CHECK(row.dim() == 3 && row.size(1) == 1, "row [B, 1, columns]");
+  ChunkAttnParams p = chunk_sizes(row.size(0), 1, H, G, dim, vdim, chunk, scale);
+  chunk_row(p, row, bias, q_w, k_w, rot, v_off, eps, cos_t, sin_t);
+  chunk_cache(p, kc, vc, row);
+  p.kv_start = starts(kv_start, row, p.B);
+  p.slot = slot_ptr(slot, row);
+  // enough key splits to fill the chip, none shorter than a step of the fullest cache
+  const int64_t groups = static_cast<int64_t>(p.B) * G * ((H / G + 15) / 16);
+  int64_t ns = std::min<int64_t>((512 + groups - 1) / groups, (p.rows + 127) / 128);
+  p.ns = static_cast<int>(std::max<int64_t>(1, std::min<int64_t>(ns, 256)));
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(row.device());
+  auto q = at::empty({p.B, 1, H, dim}, row.options()), o = at::empty({p.B, 1, H * vdim}, row.options());
+  p.q = q.data_ptr();
+  p.k = p.v = nullptr;
+  p.o = o.data_ptr();
+  at::Tensor po, ml;
+  if (p.ns > 1) {
+    po = at::empty({p.B, H, p.ns, vdim}, row.options().dtype(at::kFloat));
+    ml = at::empty({p.B, H, p.ns, 2}, po.options());
+    p.part_o = po.data_ptr<float>();
+    p.part_ml = ml.data_ptr<float>();
+  }
+  launch_chunk_prepare(bf, p, true, cur_stream(row));
+  launch_chunk_decode(bf, p, cur_stream(row));
+  return o;
+}
+
 // ---- latent attention ----
 void cache_ok(const at::Tensor& latent, const at::Tensor& ref, int64_t B, int64_t width) {
   like(latent, ref, "latent");
@@ -438,6 +824,17 @@ TORCH_LIBRARY_FRAGMENT(dla, m) {
   m.def("side_gate(Tensor z, Tensor ids, Tensor table, int off) -> Tensor");
   m.def("stream_gemm(Tensor a, Tensor w, int epi, Tensor? ssq_in, float eps, Tensor(a!)? x, Tensor? norm_w, float offset, Tensor? ids, Tensor? table, int off) -> (Tensor, Tensor)");
   m.def("relu2(Tensor u) -> Tensor");
+  m.def("post_norm(Tensor(a!) x, Tensor? delta, Tensor? bias, float alpha, Tensor w, Tensor? w2, float eps, bool bf16) -> Tensor");
+  m.def("geglu(Tensor u) -> Tensor");
+  m.def("softcap(Tensor z, float cap) -> Tensor");
+  m.def("lru_prefill(Tensor yx, Tensor bias, Tensor conv_w, Tensor conv_b, Tensor gates, Tensor gates_b, Tensor lam, float c, Tensor(a!) state, Tensor(b!) hist, Tensor? kv_start, int base) -> Tensor");
+  m.def("lru_decode(Tensor yx, Tensor bias, Tensor conv_w, Tensor conv_b, Tensor gates, Tensor gates_b, Tensor lam, float c, Tensor(a!) state, Tensor(b!) hist, Tensor slot, Tensor? kv_start) -> Tensor");
+  m.def("gla_prefill(Tensor proj, Tensor a2, Tensor a2_b, Tensor norm_w, int H, int dim, int vdim, float tau, float eps, Tensor(a!) state, Tensor? kv_start, int base) -> Tensor");
+  m.def("gla_decode(Tensor proj, Tensor a2, Tensor a2_b, Tensor norm_w, int H, int dim, int vdim, float tau, float eps, Tensor(a!) state, Tensor(b!)? cnt) -> Tensor");
+  m.def("chunk_prepare(Tensor row, Tensor bias, Tensor q_w, Tensor k_w, int H, int G, int dim, int vdim, int rot, int v_off, float eps, Tensor? kv_start, Tensor cos, Tensor sin, int base) -> (Tensor, Tensor, Tensor)");
+  m.def("chunk_prefill(Tensor q, Tensor k, Tensor v, Tensor kc, Tensor vc, int chunk, float scale, Tensor? kv_start, int base) -> Tensor");
+  m.def("chunk_store(Tensor k, Tensor v, Tensor(a!) kc, Tensor(b!) vc, int chunk, Tensor? kv_start, int base) -> ()");
+  m.def("chunk_decode(Tensor row, Tensor bias, Tensor q_w, Tensor k_w, int H, int G, int dim, int vdim, int rot, int v_off, float eps, Tensor(a!) kc, Tensor(b!) vc, int chunk, float scale, Tensor slot, Tensor? kv_start, Tensor cos, Tensor sin) -> Tensor");
   m.def("retention_prefill(Tensor qkvg, int H, int dim, int vdim, int rot, float eps, Tensor decay, Tensor(a!) state, Tensor? kv_start, Tensor cos, Tensor sin, int base) -> Tensor");
   m.def("retention_decode(Tensor qkvg, int H, int dim, int vdim, int rot, float eps, Tensor decay, Tensor(a!) state, Tensor slot, Tensor? kv_start, Tensor cos, Tensor sin, Tensor(b!)? cnt) -> Tensor");
   m.def("latent_prepare(Tensor down, Tensor q_norm_w, Tensor kv_norm_w, float eps, Tensor(a!) latent, Tensor slot, Tensor? kv_start, Tensor cos, Tensor sin) -> Tensor");
@@ -451,6 +848,17 @@ TORCH_LIBRARY_IMPL(dla, CUDA, m) {
   m.impl("side_gate", &dla::side_gate);
   m.impl("stream_gemm", &dla::stream_gemm);
   m.impl("relu2", &dla::relu2);
+  m.impl("post_norm", &dla::post_norm);
+  m.impl("geglu", &dla::geglu);
+  m.impl("softcap", &dla::softcap);
+  m.impl("lru_prefill", &dla::lru_prefill);
+  m.impl("lru_decode", &dla::lru_decode);
+  m.impl("gla_prefill", &dla::gla_prefill);
+  m.impl("gla_decode", &dla::gla_decode);
+  m.impl("chunk_prepare", &dla::chunk_prepare);
+  m.impl("chunk_prefill", &dla::chunk_prefill);
+  m.impl("chunk_store", &dla::chunk_store);
+  m.impl("chunk_decode", &dla::chunk_decode);
   m.impl("retention_prefill", &dla::retention_prefill);
   m.impl("retention_decode", &dla::retention_decode);
   m.impl("latent_prepare", &dla::latent_prepare);

@@ -18,6 +18,7 @@ import torch
 import torch.nn.functional as F
 
 from . import _ext
+from .retention import _counters
 from .stream import _rms
 
 
@@ -49,5 +50,6 @@ def decode(proj, a2, a2_b, norm_w, H: int, dim: int, vdim: int, tau: float, eps:
            base: int) -> torch.Tensor:
     """One new token per row."""
     if _ext.use_native(proj):
-        return _ext.require("mix").gla_decode(proj, a2, a2_b, norm_w, H, dim, vdim, float(tau), float(eps), state)
+        return _ext.require("mix").gla_decode(proj, a2, a2_b, norm_w, H, dim, vdim, float(tau), float(eps), state,
+                                              _counters(proj.device, proj.shape[0] * H))
     return prefill(proj, a2, a2_b, norm_w, H, dim, vdim, tau, eps, state, slot, kv_start, base)
