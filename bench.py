@@ -101,8 +101,8 @@ def parse(argv=None):
     ap.add_argument("--layers", type=int, default=None, help="debug only: override layer count "
                     "(a reduced model is NOT the benchmark config)")
     ap.add_argument("--serve", nargs="?", const="vufilorn", default=None, metavar="SIZES",
-                    help="instead of the training step: prefill / decode throughput of the per-layer design "
-                         "(vufilorn, or a comma list of presets) beside its closest attention family at equal "
+                    help="instead of the training step: prefill / decode throughput of a per-layer design "
+                         "(vufilorn, zenevik, or a comma list of presets) beside its closest models at equal "
                          "size; one JSON line per size (eval/serve_bench.py)")
     ap.add_argument("--serve-what", default="prefill,decode", help="with --serve: prefill and / or decode")
     ap.add_argument("--serve-no-peer", action="store_true", help="with --serve: the design alone")
@@ -283,7 +283,7 @@ def main(argv=None) -> int:
             raise SystemExit("--serve runs on one GPU")
         from distributed_llm_alignment_amd.eval import serve_bench
 
-        serve_bench.run(serve_bench.SIZES if args.serve == "vufilorn" else args.serve.split(","),
+        serve_bench.run(serve_bench.SIZES.get(args.serve) or args.serve.split(","),
                         tuple(args.serve_what.split(",")), peer=not args.serve_no_peer)
         return 0
     if "WORLD_SIZE" not in os.environ and args.gpus > 1:

@@ -208,16 +208,14 @@ at::Tensor relu2(const at::Tensor& u_) {
   return y;
 }
 
-// Decode projection, <= 32 rows (stream_gemm.hip): epi 0 store, 1 relu^2, 2 gate, 3 stream.
-std::tuple<at::Tensor, at::Tensor> stream_gemm(const at::Tensor& a, const at::Tensor& w, int64_t epi, const OptT& ssq_in,
-                                               double eps, OptT x, const OptT& norm_w, double offset, const OptT& ids,
-                                               const OptT& table, int64_t off) {
+// Decode projections, <= 32 rows (stream_gemm.hip)
+StreamGemmParams gemm_params(const at::Tensor& a, const at::Tensor& w, int64_t per_col, const OptT& ssq_in, double eps) {
   check_bf16(a, "a");
   check_bf16(w, "w");
   same_device(a, w);
   TORCH_CHECK(a.dim() == 2 && a.is_contiguous() && w.dim() == 2 && w.is_contiguous() && a.size(1) == w.size(1), "a [M, K], w [N, K]");
-  const int64_t M = a.size(0), N = w.size(0), K = w.size(1);
-  TORCH_CHECK(M >= 1 && M <= 32 && N >= 1 && N < (1 << 24) && K >= 8 && K < (1 << 24) && K % 8 == 0 && epi >= 0 && epi <= 3,
+  const int64_t M = a.size(0), N = w.size(0) / per_col, K = w.size(1);
+  TORCH_CHECK(M >= 1 && M <= 32 && N >= 1 && N < (1 << 24) && w.size(0) == N * per_col && K >= 8 && K < (1 << 24) && K % 8 == 0,
               "stream_gemm: 1 <= M <= 32, K % 8 == 0");
   check_aligned16(a, "a");
   check_aligned16(w, "w");
@@ -228,36 +226,51 @@ std::tuple<at::Tensor, at::Tensor> stream_gemm(const at::Tensor& a, const at::Te
   p.N = static_cast<int>(N);
   p.K = static_cast<int>(K);
   p.eps = static_cast<float>(eps);
-  p.offset = static_cast<float>(offset);
   if (ssq_in.has_value()) {
     check_f32(*ssq_in, "ssq_in");
     TORCH_CHECK(ssq_in->dim() == 2 && ssq_in->size(0) == M && ssq_in->is_contiguous() && ssq_in->device() == a.device(), "ssq_in [M, blocks]");
     p.ssq_in = ssq_in->data_ptr<float>();
     p.nssq = static_cast<int>(ssq_in->size(1));
   }
+  return p;
+}
+
+// the fp32 stream and the partial sums of squares of an epilogue that updates it; returns ssq
+at::Tensor gemm_stream(StreamGemmParams& p, const at::Tensor& a, const at::Tensor& x, const OptT& norm_w) {
+  check_f32(x, "x");
+  TORCH_CHECK(x.numel() == static_cast<int64_t>(p.M) * p.N && x.size(-1) == p.N && x.is_contiguous() && x.device() == a.device(), "x [M, N]");
+  p.x = x.data_ptr<float>();
+  if (norm_w.has_value()) {
+    vec_like(*norm_w, a, p.N, "norm_w");
+    p.norm_w = cbp(*norm_w);
+  }
+  auto ssq = at::empty({p.M, (p.N + 15) / 16}, x.options());
+  p.ssq = ssq.data_ptr<float>();
+  return ssq;
+}
+
+// epi 0 store, 1 relu^2, 2 gate, 3 stream, 5 gelu-gated unit (w = [gate; up])
+std::tuple<at::Tensor, at::Tensor> stream_gemm(const at::Tensor& a, const at::Tensor& w, int64_t epi, const OptT& ssq_in,
+                                               double eps, OptT x, const OptT& norm_w, double offset, const OptT& ids,
+                                               const OptT& table, int64_t off) {
+  TORCH_CHECK((epi >= 0 && epi <= 3) || epi == 5, "stream_gemm: epilogue");
+  StreamGemmParams p = gemm_params(a, w, epi == 5 ? 2 : 1, ssq_in, eps);
+  p.offset = static_cast<float>(offset);
   c10::hip::HIPGuardMasqueradingAsCUDA guard(a.device());
-  auto y = at::empty({M, N}, a.options());
+  auto y = at::empty({p.M, p.N}, a.options());
   p.y = bp(y);
   at::Tensor ssq;
   if (epi == 3) {
     TORCH_CHECK(x.has_value(), "stream epilogue: x");
-    check_f32(*x, "x");
-    TORCH_CHECK(x->numel() == M * N && x->size(-1) == N && x->is_contiguous() && x->device() == a.device(), "x [M, N]");
-    p.x = x->data_ptr<float>();
-    if (norm_w.has_value()) {
-      vec_like(*norm_w, a, N, "norm_w");
-      p.norm_w = cbp(*norm_w);
-    }
-    ssq = at::empty({M, (N + 15) / 16}, x->options());
-    p.ssq = ssq.data_ptr<float>();
+    ssq = gemm_stream(p, a, *x, norm_w);
   } else {
     ssq = at::empty({0}, a.options().dtype(at::kFloat));
   }
   if (epi == 2) {
     TORCH_CHECK(ids.has_value() && table.has_value(), "gate epilogue: ids, table");
-    ids_ok(*ids, a, M);
+    ids_ok(*ids, a, p.M);
     like(*table, a, "table");
-    TORCH_CHECK(table->dim() == 2 && table->stride(1) == 1 && off >= 0 && off + N <= table->size(1), "table [V, >= off + N]");
+    TORCH_CHECK(table->dim() == 2 && table->stride(1) == 1 && off >= 0 && off + p.N <= table->size(1), "table [V, >= off + N]");
     p.ids = ids->data_ptr<int64_t>();
     p.table = cbp(*table);
     p.ldt = table->stride(0);
@@ -266,6 +279,45 @@ std::tuple<at::Tensor, at::Tensor> stream_gemm(const at::Tensor& a, const at::Te
   }
   launch_stream_gemm(p, static_cast<int>(epi), cur_stream(a));
   return {y, ssq};
+}
+
+// x <- alpha x_prev + a w^T + bias (x_prev: x normed with res_ssq / res_w, or x itself); returns (bf16(x * norm_w), ssq)
+std::tuple<at::Tensor, at::Tensor> stream_gemm_post(const at::Tensor& a, const at::Tensor& w, at::Tensor x, double alpha,
+                                                    const OptT& bias, const OptT& res_ssq, const OptT& res_w,
+                                                    const at::Tensor& norm_w, double eps) {
+  StreamGemmParams p = gemm_params(a, w, 1, c10::nullopt, eps);
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(a.device());
+  auto y = at::empty({p.M, p.N}, a.options());
+  p.y = bp(y);
+  at::Tensor ssq = gemm_stream(p, a, x, norm_w);
+  p.alpha = static_cast<float>(alpha);
+  if (bias.has_value()) {
+    vec_like(*bias, a, p.N, "bias");
+    p.bias = cbp(*bias);
+  }
+  TORCH_CHECK(res_ssq.has_value() == res_w.has_value(), "res_ssq and res_w come together");
+  if (res_ssq.has_value()) {
+    check_f32(*res_ssq, "res_ssq");
+    TORCH_CHECK(res_ssq->dim() == 2 && res_ssq->size(0) == p.M && res_ssq->is_contiguous() && res_ssq->device() == a.device(), "res_ssq [M, blocks]");
+    vec_like(*res_w, a, p.N, "res_w");
+    p.res_ssq = res_ssq->data_ptr<float>();
+    p.nres = static_cast<int>(res_ssq->size(1));
+    p.res_w = cbp(*res_w);
+  }
+  launch_stream_gemm(p, 4, cur_stream(a));
+  return {y, ssq};
+}
+
+// fp32 cap * tanh(a w^T / cap)
+at::Tensor stream_gemm_cap(const at::Tensor& a, const at::Tensor& w, double cap) {
+  TORCH_CHECK(cap > 0, "cap > 0");
+  StreamGemmParams p = gemm_params(a, w, 1, c10::nullopt, 0.0);
+  c10::hip::HIPGuardMasqueradingAsCUDA guard(a.device());
+  auto y = at::empty({p.M, p.N}, a.options().dtype(at::kFloat));
+  p.yf = y.data_ptr<float>();
+  p.cap = static_cast<float>(cap);
+  launch_stream_gemm(p, 6, cur_stream(a));
+  return y;
 }
 
 // ---- retention ----
@@ -823,6 +875,8 @@ TORCH_LIBRARY_FRAGMENT(dla, m) {
   m.def("stream_norm(Tensor(a!) x, Tensor? delta, Tensor? delta_w, Tensor? inject, Tensor? w, float eps, float offset, bool bf16) -> Tensor");
   m.def("side_gate(Tensor z, Tensor ids, Tensor table, int off) -> Tensor");
   m.def("stream_gemm(Tensor a, Tensor w, int epi, Tensor? ssq_in, float eps, Tensor(a!)? x, Tensor? norm_w, float offset, Tensor? ids, Tensor? table, int off) -> (Tensor, Tensor)");
+  m.def("stream_gemm_post(Tensor a, Tensor w, Tensor(a!) x, float alpha, Tensor? bias, Tensor? res_ssq, Tensor? res_w, Tensor norm_w, float eps) -> (Tensor, Tensor)");
+  m.def("stream_gemm_cap(Tensor a, Tensor w, float cap) -> Tensor");
   m.def("relu2(Tensor u) -> Tensor");
   m.def("post_norm(Tensor(a!) x, Tensor? delta, Tensor? bias, float alpha, Tensor w, Tensor? w2, float eps, bool bf16) -> Tensor");
   m.def("geglu(Tensor u) -> Tensor");
@@ -847,6 +901,8 @@ TORCH_LIBRARY_IMPL(dla, CUDA, m) {
   m.impl("stream_norm", &dla::stream_norm);
   m.impl("side_gate", &dla::side_gate);
   m.impl("stream_gemm", &dla::stream_gemm);
+  m.impl("stream_gemm_post", &dla::stream_gemm_post);
+  m.impl("stream_gemm_cap", &dla::stream_gemm_cap);
   m.impl("relu2", &dla::relu2);
   m.impl("post_norm", &dla::post_norm);
   m.impl("geglu", &dla::geglu);

@@ -88,20 +88,21 @@ __global__ __launch_bounds__(256) void chunk_prepare_kernel(ChunkAttnParams p) {
 }
 
 // -------------------------------------------------------------------------------------- store
-// grid (min(T, chunk), G, B): the n-th last token, if it belongs to the last token's chunk
+// grid (ceil(min(T, chunk) / 16), G, B), 256 threads, 16 lanes per token: the n-th last token, if it belongs to
+// the last token's chunk
 template <typename T, int VEC>
-__global__ __launch_bounds__(64) void chunk_store_kernel(ChunkAttnParams p) {
-  const int b = blockIdx.z, hd = blockIdx.y, t = p.T - 1 - static_cast<int>(blockIdx.x);
-  const int64_t last = p.base + p.T - 1 - (p.kv_start ? p.kv_start[b] : 0), pos = last - blockIdx.x;
-  if (pos < 0 || static_cast<int64_t>(blockIdx.x) > last % p.chunk) return;
+__global__ __launch_bounds__(256) void chunk_store_kernel(ChunkAttnParams p) {
+  const int b = blockIdx.z, hd = blockIdx.y, n = blockIdx.x * 16 + (threadIdx.x >> 4), t = p.T - 1 - n;
+  const int64_t last = p.base + p.T - 1 - (p.kv_start ? p.kv_start[b] : 0), pos = last - n;
+  if (t < 0 || pos < 0 || static_cast<int64_t>(n) > last % p.chunk) return;
   const int64_t crow = pos % p.chunk, g = static_cast<int64_t>(b) * p.T + t, c = (static_cast<int64_t>(b) * p.G + hd) * p.rows + crow;
   if (crow >= p.rows) return;
   float v[VEC];
-  for (int i = threadIdx.x * VEC; i < p.dim; i += 64 * VEC) {
+  for (int i = (threadIdx.x & 15) * VEC; i < p.dim; i += 16 * VEC) {
     load_vec<T, VEC>(static_cast<const T*>(p.k) + (g * p.G + hd) * p.dim + i, v);
     store_vec<T, VEC>(static_cast<T*>(p.kc) + c * p.dim + i, v);
   }
-  for (int i = threadIdx.x * VEC; i < p.vdim; i += 64 * VEC) {
+  for (int i = (threadIdx.x & 15) * VEC; i < p.vdim; i += 16 * VEC) {
     load_vec<T, VEC>(static_cast<const T*>(p.v) + (g * p.G + hd) * p.vdim + i, v);
     store_vec<T, VEC>(static_cast<T*>(p.vc) + c * p.vdim + i, v);
   }
@@ -247,10 +248,10 @@ void prepare(const ChunkAttnParams& p, bool decode, hipStream_t st) {
 
 template <typename T>
 void store(const ChunkAttnParams& p, hipStream_t st) {
-  const dim3 g(p.T < p.chunk ? p.T : p.chunk, p.G, p.B);
+  const dim3 g(((p.T < p.chunk ? p.T : p.chunk) + 15) / 16, p.G, p.B);
   const auto al = [](const void* x) { return reinterpret_cast<uintptr_t>(x) % 16 == 0; };
-  if (p.dim % 8 == 0 && p.vdim % 8 == 0 && al(p.k) && al(p.v) && al(p.kc) && al(p.vc)) chunk_store_kernel<T, 8><<<g, 64, 0, st>>>(p);
-  else chunk_store_kernel<T, 1><<<g, 64, 0, st>>>(p);
+  if (p.dim % 8 == 0 && p.vdim % 8 == 0 && al(p.k) && al(p.v) && al(p.kc) && al(p.vc)) chunk_store_kernel<T, 8><<<g, 256, 0, st>>>(p);
+  else chunk_store_kernel<T, 1><<<g, 256, 0, st>>>(p);
 }
 
 }  // namespace

@@ -45,14 +45,37 @@ __global__ __launch_bounds__(kThreads) void gla_recurrent_kernel(GlaParams p, in
   const int grp = threadIdx.x / lpr, li = threadIdx.x % lpr, ngrp = kThreads / lpr;
   constexpr int U = 8;
   const int per = (p.vdim + p.vsplit - 1) / p.vsplit, vlo = blockIdx.z * per, vhi = min(vlo + per, p.vdim);
+  auto load_state = [&](int r0, int i, float (&s)[U][VEC]) {  // VEC state elements of U value rows
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int v = r0 + u * ngrp;
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) s[u][e] = 0.f;
+      if (v < vhi && i < p.dim) load_vec<float, VEC>(S + static_cast<int64_t>(v) * p.dim + i, s[u]);
+    }
+  };
+  const bool rank8 = p.rank % 8 == 0 && p.ld % 8 == 0 && (reinterpret_cast<uintptr_t>(p.proj) | reinterpret_cast<uintptr_t>(p.a2)) % 16 == 0 &&
+                     (2 * (Hd + Hv)) % 8 == 0;
   for (int t = 0; t < p.T; ++t) {
+    float pre[U][VEC];  // the first piece of the state is on its way while the decays are formed
+    load_state(vlo + grp, li * VEC, pre);
     const int64_t row = static_cast<int64_t>(b) * p.T + t;
     const T* in = static_cast<const T*>(p.proj) + row * p.ld;
     const bool pad = p.base + t < kv0;
     for (int i = threadIdx.x; i < p.dim; i += kThreads) {
       float z = to_f<T>(A2b[i]);
       const T *w = A2 + static_cast<int64_t>(i) * p.rank, *a = in + 2 * (Hd + Hv);
-      for (int j = 0; j < p.rank; ++j) z += to_f<T>(w[j]) * to_f<T>(a[j]);
+      if (rank8) {
+        for (int j = 0; j < p.rank; j += 8) {
+          float x[8], y[8];
+          load_vec<T, 8>(w + j, x);
+          load_vec<T, 8>(a + j, y);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) z += x[e] * y[e];
+        }
+      } else {
+        for (int j = 0; j < p.rank; ++j) z += to_f<T>(w[j]) * to_f<T>(a[j]);
+      }
       qs[i] = to_f<T>(in[h * p.dim + i]) * p.qscale;
       ks[i] = pad ? 0.f : to_f<T>(in[Hd + h * p.dim + i]);
       as[i] = pad ? 1.f : exp2f(log2_decay(z, p.inv_tau));
@@ -66,12 +89,13 @@ __global__ __launch_bounds__(kThreads) void gla_recurrent_kernel(GlaParams p, in
       for (int u = 0; u < U; ++u) acc[u] = 0.f;
       for (int i = li * VEC; i < p.dim; i += lpr * VEC) {
         float s[U][VEC];
+        if (r0 == vlo + grp && i == li * VEC) {
 #pragma unroll
-        for (int u = 0; u < U; ++u) {
-          const int v = r0 + u * ngrp;
+          for (int u = 0; u < U; ++u)
 #pragma unroll
-          for (int e = 0; e < VEC; ++e) s[u][e] = 0.f;
-          if (v < vhi && !zero) load_vec<float, VEC>(S + static_cast<int64_t>(v) * p.dim + i, s[u]);
+            for (int e = 0; e < VEC; ++e) s[u][e] = pre[u][e];
+        } else {
+          load_state(r0, i, s);
         }
 #pragma unroll
         for (int u = 0; u < U; ++u) {
@@ -79,6 +103,7 @@ __global__ __launch_bounds__(kThreads) void gla_recurrent_kernel(GlaParams p, in
           if (v >= vhi) continue;
 #pragma unroll
           for (int e = 0; e < VEC; ++e) {
+            if (zero) s[u][e] = 0.f;
             s[u][e] = as[i + e] * s[u][e] + ks[i + e] * vs[v];
             acc[u] += s[u][e] * qs[i + e];
           }

@@ -37,10 +37,18 @@ __device__ __forceinline__ f32x16 mfma32(s16x8 a, s16x8 b, f32x16 c) {
 __device__ __forceinline__ s16x4 tr4(const bf16_t* p) { return __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_s16x4*)(p)); }
 __device__ __forceinline__ s16x8 cat(s16x4 a, s16x4 b) { return s16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]}; }
 
+// log2(sigmoid(z)) = min(z, 0) log2 e - log2(1 + e^-|z|); with u = 1 + x rounded, log(1 + x) = log(u) x / (u - 1)
+__device__ __forceinline__ float log2_sigmoid(float z) {
+  constexpr float kLog2e = 1.4426950408889634f;
+  const float x = __builtin_amdgcn_exp2f(-fabsf(z) * kLog2e), u = 1.f + x, d = u - 1.f;
+  const float l = d == 0.f ? x * kLog2e : __builtin_amdgcn_logf(u) * (x * __builtin_amdgcn_rcpf(d));
+  return fminf(z, 0.f) * kLog2e - l;
+}
+
 // grid (nc, ceil(H dim / 64), B), 4 waves: wave = sub-chunk, lane = channel
 constexpr int kRank = 32;  // decay inputs staged at a time
 __global__ __launch_bounds__(kThreads) void gla_decay_kernel(GlaParams p) {
-  __shared__ float as[kC][kRank];
+  __shared__ __attribute__((aligned(16))) float as[kC][kRank];
   __shared__ float tot[4][64];
   const int b = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, Hd = p.H * p.dim;
   const int ch = blockIdx.y * 64 + lane, t0 = blockIdx.x * kC, chc = min(ch, Hd - 1);
@@ -59,18 +67,22 @@ __global__ __launch_bounds__(kThreads) void gla_decay_kernel(GlaParams p) {
     }
     __syncthreads();
     const int nr = min(kRank, p.rank - r0);
-    for (int r = 0; r < nr; ++r) {
-      const float w = bf2f(W[r0 + r]);
+    for (int r = 0; r < nr; r += 4) {
+      float w[4];
 #pragma unroll
-      for (int i = 0; i < kSub; ++i) z[i] += w * as[wave * kSub + i][r];
+      for (int e = 0; e < 4; ++e) w[e] = r + e < nr ? bf2f(W[r0 + r + e]) : 0.f;
+#pragma unroll
+      for (int i = 0; i < kSub; ++i) {
+        const f32x4 a = *reinterpret_cast<const f32x4*>(&as[wave * kSub + i][r]);
+        z[i] += w[0] * a[0] + w[1] * a[1] + w[2] * a[2] + w[3] * a[3];
+      }
     }
   }
   float l = 0.f;
 #pragma unroll
   for (int i = 0; i < kSub; ++i) {
     const int t = t0 + wave * kSub + i;
-    constexpr float kLog2e = 1.4426950408889634f;
-    if (t < p.T && p.base + t >= kv0) l += (fminf(z[i], 0.f) - log1pf(__expf(-fabsf(z[i])))) * (p.inv_tau * kLog2e);
+    if (t < p.T && p.base + t >= kv0) l += log2_sigmoid(z[i]) * p.inv_tau;
     if (t < p.T && ch < Hd) p.cum[(static_cast<int64_t>(b) * p.T + t) * Hd + ch] = l;
   }
   tot[wave][lane] = l;

@@ -4,10 +4,11 @@
 //   log a = -c r softplus(lam),  S_t = a_t S_(t-1) + sqrt(1 - a_t^2) i_t u_t,  out = S * gelu_tanh(y + bias)
 //
 // Prompt portions, three launches:
-//   gates   workgroup = (chunk of tokens, 128 channels of a gate block, sequence): the convolution of the
-//           block's channels goes to LDS, both gates' products run on MFMA with a channel per lane
-//           column, and the chunk is scanned in registers (4 tokens per lane, two shuffle steps per
-//           16 tokens). Written: the state with the chunk started at zero, and the product of decays.
+//   gates   workgroup = (chunk of tokens, gate block or 128 channels of a large one, sequence): the
+//           convolution of the block's channels goes to LDS, both gates' products run on MFMA with a
+//           channel per lane column, and the chunk is scanned in registers (4 tokens per lane, two
+//           shuffle steps per 16 tokens). Written: the state with the chunk started at zero, and the
+//           product of decays.
 //   scan    state at every chunk's start (one thread per sequence and channel); the convolution's ring
 //   output  (local state + product of decays * start state) * gelu branch, elementwise
 // Decode: one launch, workgroup = 16 channels x 16 rows, the block's input channels split over 4 waves.
@@ -20,13 +21,13 @@ namespace dla {
 namespace {
 
 constexpr int kTT = 64;    // tokens per tile
-constexpr int kNC = 128;   // channels per workgroup
+constexpr int kNC = 128;   // channels per pass
 constexpr int kKC = 256;   // gate-block inputs staged at a time
 
 template <typename T>
 constexpr int pad16() { return 16 / static_cast<int>(sizeof(T)); }
 
-__device__ __forceinline__ float sigm(float x) { return 1.f / (1.f + __expf(-x)); }
+__device__ __forceinline__ float sigm(float x) { return __builtin_amdgcn_rcpf(1.f + __expf(-x)); }
 __device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 // 1 - e^x for x <= 0, without cancellation near zero
 __device__ __forceinline__ float one_minus_exp(float x) {
@@ -38,7 +39,7 @@ __device__ __forceinline__ float one_minus_exp(float x) {
 __device__ __forceinline__ void lru_step(float zr, float zi, float u, float lam_c, float& a, float& b) {
   const float la = lam_c * sigm(zr);
   a = __expf(la);
-  b = sqrtf(one_minus_exp(2.f * la)) * sigm(zi) * u;
+  b = __builtin_amdgcn_sqrtf(one_minus_exp(2.f * la)) * sigm(zi) * u;
 }
 
 // convolution output of channel `ch` at column `col` (position pos >= 0), rounded to T; xrow(j): the raw
@@ -51,6 +52,54 @@ __device__ __forceinline__ float conv_at(const LruParams& p, int ch, int64_t pos
   for (int j = 0; j < p.taps; ++j)
     if (pos >= j) s += to_f<T>(w[p.taps - 1 - j]) * (to_f<T>(xrow(j)) + xb);
   return to_f<T>(from_f<T>(s));
+}
+
+// The same for 8 channels ch .. ch + 7 and consecutive columns, bf16, TAPS taps: `row(j)` is the raw x row of
+// column col0 + j (j >= -(TAPS - 1)), pos0 the position of column col0; emits u of n columns.
+template <int TAPS, typename F, typename G>
+__device__ __forceinline__ void conv8(const LruParams& p, int ch, int64_t pos0, int n, F row, G emit) {
+  float w[8][TAPS], xb[8], cb[8], win[TAPS][8];
+  {
+    const bf16_t* src = static_cast<const bf16_t*>(p.conv_w) + static_cast<int64_t>(ch) * TAPS;
+    bf16x8 v[TAPS];
+#pragma unroll
+    for (int i = 0; i < TAPS; ++i) v[i] = load_bf16x8(src + 8 * i);
+#pragma unroll
+    for (int e = 0; e < 8; ++e)
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) w[e][j] = bf2f(v[(e * TAPS + j) / 8][(e * TAPS + j) % 8]);
+    load_vec<bf16_t, 8>(static_cast<const bf16_t*>(p.bias) + p.W + ch, xb);
+    load_vec<bf16_t, 8>(static_cast<const bf16_t*>(p.conv_b) + ch, cb);
+  }
+  auto fetch = [&](int j, float* o) {  // biased x of column col0 + j, zero before the start
+    if (pos0 + j >= 0) {
+      load_vec<bf16_t, 8>(row(j), o);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) o[e] += xb[e];
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) o[e] = 0.f;
+    }
+  };
+#pragma unroll
+  for (int j = 0; j < TAPS - 1; ++j) fetch(j - (TAPS - 1), win[j + 1]);
+#pragma unroll 2
+  for (int t = 0; t < n; ++t) {
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) win[j][e] = win[j + 1][e];
+    fetch(t, win[TAPS - 1]);
+    float u[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      u[e] = cb[e];
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) u[e] += w[e][j] * win[j][e];
+      if (pos0 + t < 0) u[e] = 0.f;
+    }
+    emit(t, pack_bf16x8(u));
+  }
 }
 
 // 16 x KS gate-weight fragment: row `ch` of one gate block, inputs k ..
@@ -70,14 +119,15 @@ __device__ __forceinline__ typename Mma<T>::Frag gate_frag(const T* wb, int n, i
   return f;
 }
 
-// grid (nc, nb * ceil(n / 128), B), 256 threads
-template <typename T, bool VEC>
+// grid (nc, nb * ceil(n / (128 JG)), B), 256 threads; JG passes of 128 channels over a staged tile
+// (ONE: n <= kKC, the tile is staged once; JG > 1 only then). TAPS > 0: bf16, n % 8 == 0.
+template <typename T, bool VEC, int TAPS, int JG, bool ONE>
 __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   using M = Mma<T>;
   constexpr int MT = kTT / 16, NJ = kNC / 64;
-  const int nblk = (p.n + kNC - 1) / kNC;
-  const int b = blockIdx.z, blk = blockIdx.y / nblk, c0 = (blockIdx.y % nblk) * kNC;
+  const int nblk = (p.n + kNC * JG - 1) / (kNC * JG);
+  const int b = blockIdx.z, blk = blockIdx.y / nblk, c0 = (blockIdx.y % nblk) * kNC * JG;
   const int kc = min(kKC, round_up(p.n, 32)), ldu = kc + pad16<T>();
   T* us = reinterpret_cast<T*>(smem);
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
@@ -86,30 +136,37 @@ __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
   const T* Hs = static_cast<const T*>(p.hist) + static_cast<int64_t>(b) * p.taps * p.W + blk * p.n;
   const T* Wr = static_cast<const T*>(p.gates) + static_cast<int64_t>(blk) * p.n * p.n;
   const T* Wi = static_cast<const T*>(p.gates) + static_cast<int64_t>(p.nb + blk) * p.n * p.n;
-  float lam_c[NJ], rb[NJ], ib[NJ], ca[NJ], cs[NJ];
+  float lam_c[JG][NJ], rb[JG][NJ], ib[JG][NJ], ca[JG][NJ], cs[JG][NJ];
 #pragma unroll
-  for (int j = 0; j < NJ; ++j) {
-    const int ch = min(c0 + 16 * (wave + 4 * j) + r, p.n - 1);
-    lam_c[j] = -p.c * softplus(to_f<T>(static_cast<const T*>(p.lam)[blk * p.n + ch]));
-    rb[j] = to_f<T>(static_cast<const T*>(p.gates_b)[blk * p.n + ch]);
-    ib[j] = to_f<T>(static_cast<const T*>(p.gates_b)[(p.nb + blk) * p.n + ch]);
-    ca[j] = 1.f;
-    cs[j] = 0.f;
-  }
-  const int t_end = min((static_cast<int>(blockIdx.x) + 1) * p.chunk, p.T);
-  for (int t0 = blockIdx.x * p.chunk; t0 < t_end; t0 += kTT) {
-    f32x4 ar[NJ][MT], ai[NJ][MT];
-    float u[NJ][MT][4];
+  for (int q = 0; q < JG; ++q)
 #pragma unroll
-    for (int j = 0; j < NJ; ++j)
-#pragma unroll
-      for (int m = 0; m < MT; ++m) {
-        ar[j][m] = ai[j][m] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-        for (int i = 0; i < 4; ++i) u[j][m][i] = 0.f;
+    for (int j = 0; j < NJ; ++j) {
+      const int ch = min(c0 + kNC * q + 16 * (wave + 4 * j) + r, p.n - 1);
+      lam_c[q][j] = -p.c * softplus(to_f<T>(static_cast<const T*>(p.lam)[blk * p.n + ch]));
+      rb[q][j] = to_f<T>(static_cast<const T*>(p.gates_b)[blk * p.n + ch]);
+      ib[q][j] = to_f<T>(static_cast<const T*>(p.gates_b)[(p.nb + blk) * p.n + ch]);
+      ca[q][j] = 1.f;
+      cs[q][j] = 0.f;
+    }
+  auto stage = [&](int t0, int k0) {
+    if constexpr (TAPS > 0) {
+      const int ng = kc / 8, ntg = 256 / ng, per = (kTT + ntg - 1) / ntg;
+      const int k = static_cast<int>(threadIdx.x) % ng * 8, tg = threadIdx.x / ng * per;
+      const int n = min(min(per, kTT - tg), p.T - t0 - tg);  // columns of this thread that exist
+      if (tg < kTT && k0 + k < p.n && n > 0) {
+        const int64_t col = p.base + t0 + tg;
+        conv8<TAPS>(p, blk * p.n + k0 + k, col - kv0, n,
+                    [&](int j) {
+                      return t0 + tg + j >= 0 ? X + static_cast<int64_t>(t0 + tg + j) * 2 * p.W + k0 + k
+                                              : Hs + ((col + j) % TAPS) * p.W + k0 + k;
+                    },
+                    [&](int t, bf16x8 u) { store_bf16x8(us + (tg + t) * ldu + k, u); });
       }
-    for (int k0 = 0; k0 < p.n; k0 += kc) {
-      __syncthreads();  // every wave is done with the last tile
+      const bf16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
+      for (int t = max(tg, tg + max(n, 0)); t < min(tg + per, kTT); ++t) store_bf16x8(us + t * ldu + k, z);
+      if (k0 + k >= p.n && tg < kTT)
+        for (int t = tg; t < min(tg + per, kTT); ++t) store_bf16x8(us + t * ldu + k, z);
+    } else {
       for (int i = threadIdx.x; i < kTT * kc; i += 256) {
         const int t = i / kc, k = i % kc;
         float v = 0.f;
@@ -121,75 +178,106 @@ __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
           });
         us[t * ldu + k] = from_f<T>(v);
       }
-      __syncthreads();
+    }
+  };
+  const int t_end = min((static_cast<int>(blockIdx.x) + 1) * p.chunk, p.T);
+  for (int t0 = blockIdx.x * p.chunk; t0 < t_end; t0 += kTT) {
+#pragma unroll
+    for (int q = 0; q < JG; ++q) {
+      if (ONE && q == 0) {
+        __syncthreads();  // every wave is done with the last tile
+        stage(t0, 0);
+        __syncthreads();
+      }
+      f32x4 ar[NJ][MT], ai[NJ][MT];
+      float u[NJ][MT][4];
+#pragma unroll
+      for (int j = 0; j < NJ; ++j)
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+          ar[j][m] = ai[j][m] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int i = 0; i < 4; ++i) u[j][m][i] = 0.f;
+        }
+      for (int k0 = 0; k0 < (ONE ? 1 : p.n); k0 += kc) {
+        if constexpr (!ONE) {
+          __syncthreads();
+          stage(t0, k0);
+          __syncthreads();
+        }
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+          const int n0 = c0 + kNC * q + 16 * (wave + 4 * j);
+          if (n0 >= p.n) continue;
+#pragma unroll 4
+          for (int k = 0; k < kc; k += M::KS) {
+            const auto fr = gate_frag<T, VEC>(Wr, p.n, n0 + r, k0 + k + g * M::KV);
+            const auto fi = gate_frag<T, VEC>(Wi, p.n, n0 + r, k0 + k + g * M::KV);
+#pragma unroll
+            for (int m = 0; m < MT; ++m) {
+              const auto a = M::row(us + (16 * m + r) * ldu + k + g * M::KV);
+              ar[j][m] = M::mma(a, fr, ar[j][m]);
+              ai[j][m] = M::mma(a, fi, ai[j][m]);
+            }
+          }
+          const int kk = n0 + r - k0;  // this lane's own channel among the staged ones
+          if (!ONE && kk >= 0 && kk < kc)
+#pragma unroll
+            for (int m = 0; m < MT; ++m)
+#pragma unroll
+              for (int i = 0; i < 4; ++i) u[j][m][i] = to_f<T>(us[(16 * m + 4 * g + i) * ldu + kk]);
+        }
+      }
 #pragma unroll
       for (int j = 0; j < NJ; ++j) {
-        const int n0 = c0 + 16 * (wave + 4 * j);
+        const int n0 = c0 + kNC * q + 16 * (wave + 4 * j), ch = n0 + r;
         if (n0 >= p.n) continue;
-        for (int k = 0; k < kc; k += M::KS) {
-          const auto fr = gate_frag<T, VEC>(Wr, p.n, n0 + r, k0 + k + g * M::KV);
-          const auto fi = gate_frag<T, VEC>(Wi, p.n, n0 + r, k0 + k + g * M::KV);
 #pragma unroll
-          for (int m = 0; m < MT; ++m) {
-            const auto a = M::row(us + (16 * m + r) * ldu + k + g * M::KV);
-            ar[j][m] = M::mma(a, fr, ar[j][m]);
-            ai[j][m] = M::mma(a, fi, ai[j][m]);
+        for (int m = 0; m < MT; ++m) {
+          // 4 tokens of this lane: A[i], S[i] = product of decays / state since the lane's first token
+          float A[4], S[4], pa = 1.f, ps = 0.f;
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int t = t0 + 16 * m + 4 * g + i;
+            float a, x;
+            const float uv = ONE ? to_f<T>(us[(16 * m + 4 * g + i) * ldu + min(ch, kc - 1)]) : u[j][m][i];
+            lru_step(ar[j][m][i] + rb[q][j], ai[j][m][i] + ib[q][j], uv, lam_c[q][j], a, x);
+            const bool real = t < p.T && p.base + t >= kv0;
+            a = real ? a : 1.f;
+            ps = a * ps + (real ? x : 0.f);
+            pa *= a;
+            A[i] = pa;
+            S[i] = ps;
           }
-        }
-        const int kk = n0 + r - k0;  // this lane's own channel among the staged ones
-        if (kk >= 0 && kk < kc)
+          // inclusive scan over the 4 lane groups, then what comes before this lane
 #pragma unroll
-          for (int m = 0; m < MT; ++m)
-#pragma unroll
-            for (int i = 0; i < 4; ++i) u[j][m][i] = to_f<T>(us[(16 * m + 4 * g + i) * ldu + kk]);
-      }
-    }
-#pragma unroll
-    for (int j = 0; j < NJ; ++j) {
-      const int n0 = c0 + 16 * (wave + 4 * j), ch = n0 + r;
-      if (n0 >= p.n) continue;
-#pragma unroll
-      for (int m = 0; m < MT; ++m) {
-        // 4 tokens of this lane: A[i], S[i] = product of decays / state since the lane's first token
-        float A[4], S[4], pa = 1.f, ps = 0.f;
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int t = t0 + 16 * m + 4 * g + i;
-          float a = 1.f, x = 0.f;
-          if (t < p.T && p.base + t >= kv0) lru_step(ar[j][m][i] + rb[j], ai[j][m][i] + ib[j], u[j][m][i], lam_c[j], a, x);
-          ps = a * ps + x;
-          pa *= a;
-          A[i] = pa;
-          S[i] = ps;
-        }
-        // inclusive scan over the 4 lane groups, then what comes before this lane
-#pragma unroll
-        for (int o = 16; o <= 32; o <<= 1) {
-          const float qa = __shfl_up(pa, o, 64), qs = __shfl_up(ps, o, 64);
-          if (lane >= o) {
-            ps = pa * qs + ps;
-            pa *= qa;
+          for (int o = 16; o <= 32; o <<= 1) {
+            const float qa = __shfl_up(pa, o, 64), qs = __shfl_up(ps, o, 64);
+            if (lane >= o) {
+              ps = pa * qs + ps;
+              pa *= qa;
+            }
           }
-        }
-        float ea = __shfl_up(pa, 16, 64), es = __shfl_up(ps, 16, 64);
-        if (g == 0) {
-          ea = 1.f;
-          es = 0.f;
-        }
-        es = ea * cs[j] + es;
-        ea *= ca[j];
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int t = t0 + 16 * m + 4 * g + i;
-          if (t < p.T && ch < p.n) {
-            const int64_t at = (static_cast<int64_t>(b) * p.T + t) * p.W + blk * p.n + ch;
-            p.cum[at] = ea * A[i];
-            p.loc[at] = A[i] * es + S[i];
+          float ea = __shfl_up(pa, 16, 64), es = __shfl_up(ps, 16, 64);
+          if (g == 0) {
+            ea = 1.f;
+            es = 0.f;
           }
+          es = ea * cs[q][j] + es;
+          ea *= ca[q][j];
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int t = t0 + 16 * m + 4 * g + i;
+            if (t < p.T && ch < p.n) {
+              const int64_t at = (static_cast<int64_t>(b) * p.T + t) * p.W + blk * p.n + ch;
+              p.cum[at] = ea * A[i];
+              p.loc[at] = A[i] * es + S[i];
+            }
+          }
+          const float la = __shfl(pa, 48 + r, 64), ls = __shfl(ps, 48 + r, 64);
+          cs[q][j] = la * cs[q][j] + ls;
+          ca[q][j] *= la;
         }
-        const float la = __shfl(pa, 48 + r, 64), ls = __shfl(ps, 48 + r, 64);
-        cs[j] = la * cs[j] + ls;
-        ca[j] *= la;
       }
     }
   }
@@ -254,9 +342,9 @@ __global__ __launch_bounds__(256) void lru_output_kernel(LruParams p) {
   }
 }
 
-// grid (nb * ceil(n / 16), ceil(B / 16)), 256 threads
+// grid (nb * ceil(n / 16), ceil(B / 16)), 256 threads. TAPS > 0: bf16, n % 8 == 0.
 constexpr int kDK = 1024;  // gate-block inputs staged at a time
-template <typename T, bool VEC>
+template <typename T, bool VEC, int TAPS>
 __global__ __launch_bounds__(256) void lru_decode_kernel(LruParams p) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   __shared__ float red[2][4][4][64];
@@ -265,35 +353,75 @@ __global__ __launch_bounds__(256) void lru_decode_kernel(LruParams p) {
   const int kc = min(kDK, round_up(p.n, 32)), ldu = kc + pad16<T>();
   T* us = reinterpret_cast<T*>(smem);
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63, r = lane & 15, g = lane >> 4;
-  const int64_t col = p.slot[0];
   const int nr = min(16, p.B - b0);
   const T* Wr = static_cast<const T*>(p.gates) + static_cast<int64_t>(blk) * p.n * p.n;
   const T* Wi = static_cast<const T*>(p.gates) + static_cast<int64_t>(p.nb + blk) * p.n * p.n;
   const T* YX = static_cast<const T*>(p.yx);
   T* Hs = static_cast<T*>(p.hist);
+  const int ti = 4 * g + wave, ch = n0 + r;  // this thread's output: row ti, channel ch
+  // the first weights leave before the convolution; the rest of the thread's operands with them
+  constexpr int UK = 2;
+  typename M::Frag fr[UK], fi[UK];
+#pragma unroll
+  for (int q = 0; q < UK; ++q) {
+    const int k = (wave + 4 * q) * M::KS + g * M::KV;
+    fr[q] = gate_frag<T, VEC>(Wr, p.n, ch, k);
+    fi[q] = gate_frag<T, VEC>(Wi, p.n, ch, k);
+  }
+  const bool out = ti < nr && ch < p.n;
+  const int c = blk * p.n + min(ch, p.n - 1), bo = b0 + min(ti, nr - 1);
+  const int64_t at = static_cast<int64_t>(bo) * p.W + c;
+  const float br = to_f<T>(static_cast<const T*>(p.gates_b)[c]), bi = to_f<T>(static_cast<const T*>(p.gates_b)[p.W + c]);
+  const float lam = to_f<T>(static_cast<const T*>(p.lam)[c]), S0 = p.state[at];
+  const T y0 = YX[static_cast<int64_t>(bo) * 2 * p.W + c], x0 = YX[static_cast<int64_t>(bo) * 2 * p.W + p.W + c];
+  const float yb = to_f<T>(static_cast<const T*>(p.bias)[c]);
+  const int64_t col = p.slot[0];
   f32x4 ar = {0.f, 0.f, 0.f, 0.f}, ai = ar;
-  float uo = 0.f;  // this thread's output: row ti, channel n0 + r
-  const int ti = 4 * g + wave, ch = n0 + r;
+  float uo = 0.f;
   for (int k0 = 0; k0 < p.n; k0 += kc) {
     if (k0) __syncthreads();
-    for (int i = threadIdx.x; i < 16 * kc; i += 256) {
-      const int m = i / kc, k = i % kc;
-      float v = 0.f;
-      if (m < nr && k0 + k < p.n) {
-        const int c = blk * p.n + k0 + k, b = b0 + m;
-        const int64_t pos = col - (p.kv_start ? p.kv_start[b] : 0);
-        v = conv_at<T>(p, c, pos, [&](int j) {
-          return j == 0 ? YX[static_cast<int64_t>(b) * 2 * p.W + p.W + c]
-                        : Hs[(static_cast<int64_t>(b) * p.taps + (col - j) % p.taps) * p.W + c];
-        });
+    if constexpr (TAPS > 0) {
+      for (int i = threadIdx.x; i < 16 * (kc / 8); i += 256) {
+        const int m = i / (kc / 8), k = i % (kc / 8) * 8, b = b0 + m;
+        if (m < nr && k0 + k < p.n) {
+          const int cc = blk * p.n + k0 + k;
+          conv8<TAPS>(p, cc, col - (p.kv_start ? p.kv_start[b] : 0), 1,
+                      [&](int j) {
+                        return j == 0 ? YX + static_cast<int64_t>(b) * 2 * p.W + p.W + cc
+                                      : Hs + (static_cast<int64_t>(b) * TAPS + (col + j) % TAPS) * p.W + cc;
+                      },
+                      [&](int, bf16x8 u) { store_bf16x8(us + m * ldu + k, u); });
+        } else {
+          store_bf16x8(us + m * ldu + k, bf16x8{0, 0, 0, 0, 0, 0, 0, 0});
+        }
       }
-      us[m * ldu + k] = from_f<T>(v);
+    } else {
+      for (int i = threadIdx.x; i < 16 * kc; i += 256) {
+        const int m = i / kc, k = i % kc;
+        float v = 0.f;
+        if (m < nr && k0 + k < p.n) {
+          const int cc = blk * p.n + k0 + k, b = b0 + m;
+          v = conv_at<T>(p, cc, col - (p.kv_start ? p.kv_start[b] : 0), [&](int j) {
+            return j == 0 ? YX[static_cast<int64_t>(b) * 2 * p.W + p.W + cc]
+                          : Hs[(static_cast<int64_t>(b) * p.taps + (col - j) % p.taps) * p.W + cc];
+          });
+        }
+        us[m * ldu + k] = from_f<T>(v);
+      }
     }
     __syncthreads();
-    for (int k = wave * M::KS; k < kc; k += 4 * M::KS) {
+    int q = 0;
+#pragma unroll
+    for (int k = wave * M::KS; k < kc; k += 4 * M::KS, ++q) {
       const auto a = M::row(us + r * ldu + k + g * M::KV);
-      ar = M::mma(a, gate_frag<T, VEC>(Wr, p.n, ch, k0 + k + g * M::KV), ar);
-      ai = M::mma(a, gate_frag<T, VEC>(Wi, p.n, ch, k0 + k + g * M::KV), ai);
+      const bool have = k0 == 0 && q < UK;
+      auto wr = q == 0 ? fr[0] : fr[1], wi = q == 0 ? fi[0] : fi[1];
+      if (!have) {
+        wr = gate_frag<T, VEC>(Wr, p.n, ch, k0 + k + g * M::KV);
+        wi = gate_frag<T, VEC>(Wi, p.n, ch, k0 + k + g * M::KV);
+      }
+      ar = M::mma(a, wr, ar);
+      ai = M::mma(a, wi, ai);
     }
     if (ch - k0 >= 0 && ch - k0 < kc) uo = to_f<T>(us[ti * ldu + ch - k0]);
   }
@@ -303,25 +431,23 @@ __global__ __launch_bounds__(256) void lru_decode_kernel(LruParams p) {
     red[1][wave][i][lane] = ai[i];
   }
   __syncthreads();
-  if (ti >= nr || ch >= p.n) return;  // (register i = wave of every wave's tile: row 4 g + wave)
-  float zr = 0.f, zi = 0.f;
+  if (!out) return;  // (register i = wave of every wave's tile: row 4 g + wave)
+  float zr = br, zi = bi;
 #pragma unroll
   for (int w = 0; w < 4; ++w) {
     zr += red[0][w][wave][lane];
     zi += red[1][w][wave][lane];
   }
-  const int c = blk * p.n + ch, b = b0 + ti;
-  zr += to_f<T>(static_cast<const T*>(p.gates_b)[blk * p.n + ch]);
-  zi += to_f<T>(static_cast<const T*>(p.gates_b)[(p.nb + blk) * p.n + ch]);
   float a, x;
-  lru_step(zr, zi, uo, -p.c * softplus(to_f<T>(static_cast<const T*>(p.lam)[c])), a, x);
-  const int64_t at = static_cast<int64_t>(b) * p.W + c;
-  const float S = a * p.state[at] + x;
+  lru_step(zr, zi, uo, -p.c * softplus(lam), a, x);
+  const float S = a * S0 + x;
   p.state[at] = S;
-  const T* in = YX + static_cast<int64_t>(b) * 2 * p.W;
-  Hs[(static_cast<int64_t>(b) * p.taps + col % p.taps) * p.W + c] = in[p.W + c];
-  static_cast<T*>(p.out)[at] = from_f<T>(S * gelu_tanh(to_f<T>(in[c]) + to_f<T>(static_cast<const T*>(p.bias)[c])));
+  Hs[(static_cast<int64_t>(bo) * p.taps + col % p.taps) * p.W + c] = x0;
+  static_cast<T*>(p.out)[at] = from_f<T>(S * gelu_tanh(to_f<T>(y0) + yb));
 }
+
+// passes of 128 channels per workgroup
+int lru_passes(const LruParams& p) { return p.n > kNC && p.n <= kKC ? 2 : 1; }
 
 template <typename K>
 void allow_lds(K kernel, int64_t bytes) {
@@ -330,22 +456,43 @@ void allow_lds(K kernel, int64_t bytes) {
                               static_cast<int>(bytes));
 }
 
-template <typename T>
-bool gates_vec(const LruParams& p) {
-  return p.n % 8 == 0 && reinterpret_cast<uintptr_t>(p.gates) % 16 == 0;
+bool gates_vec(const LruParams& p) { return p.n % 8 == 0 && reinterpret_cast<uintptr_t>(p.gates) % 16 == 0; }
+
+// taps of the vectorised convolution, 0: element by element
+int conv_taps(bool bf16, const LruParams& p) {
+  const auto al = [](const void* x) { return reinterpret_cast<uintptr_t>(x) % 16 == 0; };
+  const bool ok = bf16 && gates_vec(p) && p.taps >= 2 && p.taps <= 4 && al(p.yx) && al(p.bias) && al(p.conv_w) && al(p.conv_b) &&
+                  al(p.hist);
+  return ok ? p.taps : 0;
+}
+
+template <typename T, bool VEC, int TAPS, int JG, bool ONE>
+void gates(const LruParams& p, hipStream_t st) {
+  const dim3 g(p.nc, p.nb * ((p.n + kNC * JG - 1) / (kNC * JG)), p.B);
+  const int kc = p.n < kKC ? round_up(p.n, 32) : kKC;
+  const int64_t lds = static_cast<int64_t>(sizeof(T)) * kTT * (kc + pad16<T>());
+  allow_lds(lru_gates_kernel<T, VEC, TAPS, JG, ONE>, lds);
+  lru_gates_kernel<T, VEC, TAPS, JG, ONE><<<g, 256, lds, st>>>(p);
+}
+template <typename T, bool VEC, int TAPS>
+void gates(const LruParams& p, hipStream_t st) {
+  if (lru_passes(p) == 2) gates<T, VEC, TAPS, 2, true>(p, st);
+  else if (p.n <= kKC) gates<T, VEC, TAPS, 1, true>(p, st);
+  else gates<T, VEC, TAPS, 1, false>(p, st);
 }
 
 template <typename T>
 void prefill(const LruParams& p, hipStream_t st) {
-  const dim3 g(p.nc, p.nb * ((p.n + kNC - 1) / kNC), p.B);
-  const int kc = p.n < kKC ? round_up(p.n, 32) : kKC;
-  const int64_t lds = static_cast<int64_t>(sizeof(T)) * kTT * (kc + pad16<T>());
-  if (gates_vec<T>(p)) {
-    allow_lds(lru_gates_kernel<T, true>, lds);
-    lru_gates_kernel<T, true><<<g, 256, lds, st>>>(p);
+  if constexpr (sizeof(T) == 2) {
+    const int taps = conv_taps(true, p);
+    if (taps == 4) gates<T, true, 4>(p, st);
+    else if (taps == 3) gates<T, true, 3>(p, st);
+    else if (taps == 2) gates<T, true, 2>(p, st);
+    else if (gates_vec(p)) gates<T, true, 0>(p, st);
+    else gates<T, false, 0>(p, st);
   } else {
-    allow_lds(lru_gates_kernel<T, false>, lds);
-    lru_gates_kernel<T, false><<<g, 256, lds, st>>>(p);
+    if (gates_vec(p)) gates<T, true, 0>(p, st);
+    else gates<T, false, 0>(p, st);
   }
   lru_scan_kernel<T><<<dim3((p.W + 63) / 64, p.B), 64, 0, st>>>(p);
   const auto al = [](const void* x) { return reinterpret_cast<uintptr_t>(x) % 16 == 0; };
@@ -356,17 +503,27 @@ void prefill(const LruParams& p, hipStream_t st) {
     lru_output_kernel<T, 1><<<dim3((p.W + 255) / 256, ty, p.B), 256, 0, st>>>(p);
 }
 
-template <typename T>
-void decode(const LruParams& p, hipStream_t st) {
+template <typename T, bool VEC, int TAPS>
+void step(const LruParams& p, hipStream_t st) {
   const dim3 g(p.nb * ((p.n + 15) / 16), (p.B + 15) / 16);
   const int kc = p.n < kDK ? round_up(p.n, 32) : kDK;
   const int64_t lds = static_cast<int64_t>(sizeof(T)) * 16 * (kc + pad16<T>());
-  if (gates_vec<T>(p)) {
-    allow_lds(lru_decode_kernel<T, true>, lds);
-    lru_decode_kernel<T, true><<<g, 256, lds, st>>>(p);
+  allow_lds(lru_decode_kernel<T, VEC, TAPS>, lds);
+  lru_decode_kernel<T, VEC, TAPS><<<g, 256, lds, st>>>(p);
+}
+
+template <typename T>
+void decode(const LruParams& p, hipStream_t st) {
+  if constexpr (sizeof(T) == 2) {
+    const int taps = conv_taps(true, p);
+    if (taps == 4) step<T, true, 4>(p, st);
+    else if (taps == 3) step<T, true, 3>(p, st);
+    else if (taps == 2) step<T, true, 2>(p, st);
+    else if (gates_vec(p)) step<T, true, 0>(p, st);
+    else step<T, false, 0>(p, st);
   } else {
-    allow_lds(lru_decode_kernel<T, false>, lds);
-    lru_decode_kernel<T, false><<<g, 256, lds, st>>>(p);
+    if (gates_vec(p)) step<T, true, 0>(p, st);
+    else step<T, false, 0>(p, st);
   }
 }
 
@@ -374,7 +531,8 @@ void decode(const LruParams& p, hipStream_t st) {
 
 // tokens per chunk: enough workgroups for the chip, few chunks to scan
 int lru_chunk(const LruParams& p) {
-  const int64_t per = static_cast<int64_t>(p.nb) * ((p.n + kNC - 1) / kNC) * p.B;
+  const int nc = kNC * lru_passes(p);
+  const int64_t per = static_cast<int64_t>(p.nb) * ((p.n + nc - 1) / nc) * p.B;
   int c = 4 * kTT;
   while (c > kTT && per * ((p.T + c - 1) / c) < 1024) c /= 2;
   return c;

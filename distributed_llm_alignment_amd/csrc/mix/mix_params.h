@@ -137,6 +137,13 @@ struct StreamGemmParams {
   const uint16_t* norm_w;  // stream epilogue: the next norm's weight, or nullptr
   float offset;
   float* ssq;              // stream epilogue: [M, ceil(N / 16)]
+  float alpha;             // post epilogue: x <- alpha x_prev + . + bias
+  const float* res_ssq;    // post epilogue: x holds a sum before its norm; [M, nres] partial sums of squares, or nullptr
+  int nres;
+  const uint16_t* res_w;   // post epilogue: [N] weight of that norm
+  const uint16_t* bias;    // post epilogue: [N], or nullptr
+  float* yf;               // cap epilogue: fp32 [M, N]
+  float cap;
   const int64_t* ids;      // gate epilogue: [M]
   const uint16_t* table;
   int64_t ldt, off, vocab;

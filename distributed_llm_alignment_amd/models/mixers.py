@@ -48,7 +48,9 @@ class Stream:
     delta_w: Optional[torch.Tensor] = None  # plain RMS norm of delta with this weight before the add
     inject: Optional[torch.Tensor] = None
     post: Optional[PostNorm] = None
-    ssq: Optional[torch.Tensor] = None  # fused decode: x is the sum before `post`, these its partial sums of squares
+    # fused decode: x is the sum before `post`, these its partial sums of squares and its rows x * post.w
+    ssq: Optional[torch.Tensor] = None
+    rows: Optional[torch.Tensor] = None
 
     def norm(self, w, eps: float, offset: float, dtype) -> torch.Tensor:
         """Fold the pending update into x and return the normed rows."""
@@ -68,7 +70,7 @@ class Stream:
             y, self.x = ops.post_norm(self.x, None, None, 1.0, p.w, w2, p.eps, dtype)
         else:
             y, self.x = ops.post_norm(self.x, self.delta, p.bias, p.alpha, p.w, w2, p.eps, dtype)
-        self.delta = self.post = self.ssq = None
+        self.delta = self.post = self.ssq = self.rows = None
         return y
 
     def last_norm(self, w, eps: float, offset: float, dtype) -> torch.Tensor:
@@ -413,8 +415,35 @@ class PostNormLayer(nn.Module):
             self.mlp = MLP(dataclasses.replace(cfg, intermediate_size=spec["mlp"]["ff"]), device, dtype)
         self.recompute = None
 
+    def fused_ok(self, rows: int) -> bool:
+        """A decode step of this layer can run on the fused projections (norm in front, sum and norm /
+        gated unit behind)."""
+        ws = self.mix.matrices()
+        if self.mlp is not None:
+            ws += (self.mlp.up_proj, self.mlp.down_proj)
+        return ops.stream.fused_ok(rows, self.ln1_w.dtype, *ws)
+
+    def decode_fused(self, s: Stream, cache, slot: CacheSlot) -> Stream:
+        cfg, st = self.cfg, ops.stream
+        eps, alpha = cfg.norm_eps, cfg.postln_alpha
+        if s.ssq is None:
+            h, prev = s.cast(eps, self.ln1_w.dtype), (None, None)
+        else:
+            h, prev = s.rows, (s.ssq, s.post.w)
+        a = self.mix.mix(st.fused_linear(h, self.mix.in_proj, prev[0], eps), cache, slot)
+        w = self.ln1_w
+        h, ssq = st.fused_post(a, self.mix.o_proj, s.x, alpha, self.mix.o_bias, *prev, w, eps)
+        if self.mlp is not None:
+            m = st.fused_geglu(h, self.mlp.up_proj, ssq, eps)
+            h, ssq = st.fused_post(m, self.mlp.down_proj, s.x, alpha, None, ssq, w, self.ln2_w, eps)
+            w = self.ln2_w
+        s.rows, s.ssq, s.post = h, ssq, PostNorm(w, alpha, eps)
+        return s
+
     def forward(self, s: Stream, ids: torch.Tensor, side_embed, cache, slot: CacheSlot) -> Stream:
         cfg, dt = self.cfg, self.ln1_w.dtype
+        if ids.shape[1] == 1 and not torch.is_grad_enabled() and self.fused_ok(ids.shape[0]):
+            return self.decode_fused(s, cache, slot)
         a = self.mix.mix(ops.stream_linear(s.cast(cfg.norm_eps, dt), self.mix.in_proj), cache, slot)
         s.delta = ops.stream_linear(a, self.mix.o_proj)
         s.post = PostNorm(self.ln1_w, cfg.postln_alpha, cfg.norm_eps, self.mix.o_bias)

@@ -617,8 +617,7 @@ class CausalLM(nn.Module):
 
     def logits(self, hidden: torch.Tensor) -> torch.Tensor:
         if self.cfg.layer_specs is not None:
-            lg = ops.head_logits(hidden, self.head_weight)
-            return ops.softcap(lg, self.cfg.logit_softcap) if self.cfg.logit_softcap else lg
+            return ops.head_logits(hidden, self.head_weight, self.cfg.logit_softcap)
         lg = None
         if self.lm_head_bias is None and self.vocab_parallel is None:
             lg = ops.decode.head_f8(hidden, self.head_weight)  # fp8 decode mode only

@@ -102,11 +102,15 @@ def stream_linear(x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
     return F.linear(x, w)
 
 
-def head_logits(h: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
+def head_logits(h: torch.Tensor, w: torch.Tensor, cap: float = 0.0) -> torch.Tensor:
+    """h w^T, with a soft cap cap * tanh(. / cap) in fp32."""
     rows = h.numel() // h.shape[-1]
     if h.is_cuda and fused_ok(rows, h.dtype, w) and not torch.is_grad_enabled():
+        if cap:
+            return _ext.require("mix").stream_gemm_cap(_rows(h), w, float(cap)).view(*h.shape[:-1], w.shape[0])
         return fused_linear(h, w)
-    return F.linear(h, w)
+    z = F.linear(h, w)
+    return softcap(z, cap) if cap else z
 
 
 # ------------------------------------------------------------------------ fused decode projections
@@ -116,7 +120,7 @@ STREAM_FUSED = os.environ.get("DLA_STREAM_FUSED", "1") != "0"
 # (17 .. 32 rows run too, but every workgroup re-reads all of a for its 16 columns: at 32 rows that is
 # more L2 traffic than the weights, and the library's GEMMs are ahead)
 STREAM_FUSED_ROWS = int(os.environ.get("DLA_STREAM_FUSED_ROWS", "16"))
-_STORE, _RELU2, _GATE, _STREAM = range(4)
+_STORE, _RELU2, _GATE, _STREAM, _GEGLU = 0, 1, 2, 3, 5  # (4, 6: ops of their own)
 
 
 def fused_ok(rows: int, dtype: torch.dtype, *weights: torch.Tensor) -> bool:
@@ -137,6 +141,21 @@ def fused_linear(a: torch.Tensor, w: torch.Tensor, ssq: Optional[torch.Tensor] =
     y, _ = _ext.require("mix").stream_gemm(_rows(a), w, _RELU2 if relu2 else _STORE, ssq, float(eps), None, None, 0.0,
                                            None, None, 0)
     return y.view(*a.shape[:-1], w.shape[0])
+
+
+def fused_geglu(a: torch.Tensor, w: torch.Tensor, ssq: Optional[torch.Tensor] = None, eps: float = 0.0) -> torch.Tensor:
+    """geglu(rowscale * (a W^T)), W = [gate; up]."""
+    y, _ = _ext.require("mix").stream_gemm(_rows(a), w, _GEGLU, ssq, float(eps), None, None, 0.0, None, None, 0)
+    return y.view(*a.shape[:-1], w.shape[0] // 2)
+
+
+def fused_post(a: torch.Tensor, w: torch.Tensor, x: torch.Tensor, alpha: float, bias: Optional[torch.Tensor],
+               res_ssq: Optional[torch.Tensor], res_w: Optional[torch.Tensor], norm_w: torch.Tensor, eps: float):
+    """x <- alpha x_prev + a W^T + bias (fp32, in place), x_prev = x or, with `res_ssq` (x's partial sums of
+    squares) and `res_w`, RMSNorm(x) * res_w. Returns (x * norm_w in bf16, x's partial sums of squares):
+    the next projection sees RMSNorm(x) * norm_w through its row scale."""
+    y, ssq = _ext.require("mix").stream_gemm_post(_rows(a), w, x, float(alpha), bias, res_ssq, res_w, norm_w, float(eps))
+    return y.view(*a.shape[:-1], w.shape[0]), ssq
 
 
 def fused_gate(a: torch.Tensor, w: torch.Tensor, ids: torch.Tensor, side_embed: torch.Tensor, off: int) -> torch.Tensor:

@@ -248,6 +248,36 @@ def test_geglu_softcap(F, where):
     rel(got, O.softcap(f64(z), 5.0), where, 2e-6, 2e-6)
 
 
+@GPU
+@pytest.mark.parametrize("M", [1, 5, 16, 17, 32])
+@pytest.mark.parametrize("N,K", [(50, 72), (256, 2048), (2048, 1024), (33, 264)])
+def test_fused_decode_projections(M, N, K):
+    """Sum and norm behind a projection (with and without a norm pending on x), the gated unit and the
+    soft cap, against float64."""
+    where = ("cuda", torch.bfloat16)
+    a, w, st = rnd(where, M, 1, K), rnd(where, N, K, scale=K ** -0.5), ops.stream
+    want = f64(a)[:, 0] @ f64(w).T
+    x, nw, rw, bias = torch.randn(M, 1, N, device="cuda") * 2, rnd(where, N), rnd(where, N, seed=1), rnd(where, N, seed=2)
+    ssq = torch.stack([p.pow(2).sum(-1) for p in x[:, 0].split(16, -1)], -1).contiguous()
+    for res, rwt, b in ((None, None, None), (ssq, rw, None), (ssq, rw, bias)):
+        xi = x.clone()
+        h, sq = st.fused_post(a, w, xi, 1.6, b, res, rwt, nw, 1e-3)
+        prev = f64(x)[:, 0] if res is None else O.rms(f64(x)[:, 0], 1e-3) * f64(rw)
+        xw = 1.6 * prev + want + (0 if b is None else f64(b))
+        rel(xi[:, 0], xw, where, b16=2e-5)  # the stream is fp32
+        rel(sq.sum(1), (xw ** 2).sum(1), where, b16=2e-5)
+        rel(h[:, 0], xw * f64(nw), where)
+    u = rnd(where, 2 * N, K, seed=4, scale=K ** -0.5)
+    scale = 1 / torch.sqrt(f64(ssq).sum(1, keepdim=True) / K + 1e-3)
+    gu = f64(a)[:, 0] @ f64(u).T
+    rel(st.fused_geglu(a, u)[:, 0], O.gelu_tanh(gu[:, :N]) * gu[:, N:], where)
+    gu = gu * scale
+    rel(st.fused_geglu(a, u, ssq, 1e-3)[:, 0], O.gelu_tanh(gu[:, :N]) * gu[:, N:], where)
+    got = ops.head_logits(a * 4, w, 3.0)
+    assert got.dtype == torch.float32
+    rel(got[:, 0], O.softcap(4 * want, 3.0), where)
+
+
 def _lru_case(where, W, nb, taps, seed=0):
     P = O.weights(O.config(8, 4, [(O.lru(W, nb, taps), None)]), seed=seed + W)
     t = {k.split("mix.")[1]: v.to(where[0], where[1]) for k, v in P.items() if ".mix." in k}
@@ -265,7 +295,7 @@ def _lru_oracle(yx, t, W, u_dtype):
 
 
 @pytest.mark.parametrize("where", WHERE)
-@pytest.mark.parametrize("W,nb,taps", [(64, 4, 4), (35, 5, 3), (7, 7, 1), (320, 2, 6), (512, 1, 4)])
+@pytest.mark.parametrize("W,nb,taps", [(64, 4, 4), (35, 5, 3), (7, 7, 1), (320, 2, 6), (512, 2, 4), (200, 1, 2), (312, 1, 3)])
 def test_lru_alone(W, nb, taps, where):
     """Tiles and chunks of tokens, a second portion, one shorter than the convolution, decode; a padded
     row whose padding holds NaN, and stale state and history that a fresh sequence must not see."""
