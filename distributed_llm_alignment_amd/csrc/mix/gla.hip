@@ -27,7 +27,7 @@ __device__ __forceinline__ float log2_decay(float z, float inv_tau) {
 // grid (H, B, vsplit); a row of the state (one v) belongs to a group of `lpr` lanes, each lane to
 // VEC-element pieces of it
 template <typename T, int VEC>
-__global__ __launch_bounds__(kThreads) void gla_recurrent_kernel(GlaParams p, int lpr) {
+__global__ __launch_bounds__(kThreads, 4) void gla_recurrent_kernel(GlaParams p, int lpr) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   __shared__ float scratch[kThreads / 64];
   const int d4 = round_up(p.dim, 4);
@@ -43,7 +43,7 @@ __global__ __launch_bounds__(kThreads) void gla_recurrent_kernel(GlaParams p, in
   const T* A2b = static_cast<const T*>(p.a2_b) + h * p.dim;
   float* S = p.state + (static_cast<int64_t>(b) * p.H + h) * p.vdim * p.dim;
   const int grp = threadIdx.x / lpr, li = threadIdx.x % lpr, ngrp = kThreads / lpr;
-  constexpr int U = 8;
+  constexpr int U = 4;
   const int per = (p.vdim + p.vsplit - 1) / p.vsplit, vlo = blockIdx.z * per, vhi = min(vlo + per, p.vdim);
   auto load_state = [&](int r0, int i, float (&s)[U][VEC]) {  // VEC state elements of U value rows
 #pragma unroll

@@ -45,48 +45,61 @@ __device__ __forceinline__ float log2_sigmoid(float z) {
   return fminf(z, 0.f) * kLog2e - l;
 }
 
-// grid (nc, ceil(H dim / 64), B), 4 waves: wave = sub-chunk, lane = channel
-constexpr int kRank = 32;  // decay inputs staged at a time
+// grid (nc, ceil(H dim / 64), B), 4 waves: wave = sub-chunk of tokens, 2 tiles of 32 channels
 __global__ __launch_bounds__(kThreads) void gla_decay_kernel(GlaParams p) {
-  __shared__ __attribute__((aligned(16))) float as[kC][kRank];
   __shared__ float tot[4][64];
-  const int b = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, Hd = p.H * p.dim;
-  const int ch = blockIdx.y * 64 + lane, t0 = blockIdx.x * kC, chc = min(ch, Hd - 1);
-  const int kv0 = p.kv_start ? p.kv_start[b] : 0;
-  const bf16_t* A = static_cast<const bf16_t*>(p.proj) + (static_cast<int64_t>(b) * p.T + t0) * p.ld + 2 * (Hd + p.H * p.vdim);
-  const bf16_t* W = static_cast<const bf16_t*>(p.a2) + static_cast<int64_t>(chc) * p.rank;
-  float z[kSub];
-  const float bias = bf2f(static_cast<const bf16_t*>(p.a2_b)[chc]);
+  const int b = blockIdx.z, lane = threadIdx.x & 63, wave = threadIdx.x >> 6, Hd = p.H * p.dim, c32 = lane & 31, g = lane >> 5;
+  const int t0 = blockIdx.x * kC + wave * kSub, kv0 = p.kv_start ? p.kv_start[b] : 0;
+  const int64_t row0 = static_cast<int64_t>(b) * p.T;
+  const bf16_t* A = static_cast<const bf16_t*>(p.proj) + (row0 + min(t0 + c32, p.T - 1)) * p.ld + 2 * (Hd + p.H * p.vdim);
+  const bf16_t* W = static_cast<const bf16_t*>(p.a2);
+  f32x16 z[2];
+  float bias[2];
 #pragma unroll
-  for (int i = 0; i < kSub; ++i) z[i] = bias;
-  for (int r0 = 0; r0 < p.rank; r0 += kRank) {
-    __syncthreads();
-    for (int i = threadIdx.x; i < kC * kRank; i += kThreads) {
-      const int t = i / kRank, r = i % kRank;
-      as[t][r] = t0 + t < p.T && r0 + r < p.rank ? bf2f(A[t * p.ld + r0 + r]) : 0.f;
+  for (int n = 0; n < 2; ++n) {
+    bias[n] = bf2f(static_cast<const bf16_t*>(p.a2_b)[min(static_cast<int>(blockIdx.y) * 64 + 32 * n + c32, Hd - 1)]);
+#pragma unroll
+    for (int i = 0; i < 16; ++i) z[n][i] = 0.f;
+  }
+  for (int k0 = 0; k0 < p.rank; k0 += 16) {  // (rank % 8 == 0)
+    const int k = k0 + 8 * g;
+    const bool in = k < p.rank;
+    s16x8 a = Mma<bf16_t>::zero(), w[2] = {a, a};
+    if (in) {
+      a = Mma<bf16_t>::row(A + k);
+#pragma unroll
+      for (int n = 0; n < 2; ++n)
+        w[n] = Mma<bf16_t>::row(W + static_cast<int64_t>(min(static_cast<int>(blockIdx.y) * 64 + 32 * n + c32, Hd - 1)) * p.rank + k);
     }
-    __syncthreads();
-    const int nr = min(kRank, p.rank - r0);
-    for (int r = 0; r < nr; r += 4) {
-      float w[4];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) w[e] = r + e < nr ? bf2f(W[r0 + r + e]) : 0.f;
+    for (int n = 0; n < 2; ++n) z[n] = mfma32(a, w[n], z[n]);
+  }
 #pragma unroll
-      for (int i = 0; i < kSub; ++i) {
-        const f32x4 a = *reinterpret_cast<const f32x4*>(&as[wave * kSub + i][r]);
-        z[i] += w[0] * a[0] + w[1] * a[1] + w[2] * a[2] + w[3] * a[3];
+  for (int n = 0; n < 2; ++n) {
+    const int ch = blockIdx.y * 64 + 32 * n + c32;
+    // this lane's tokens are 8 u + 4 g + e: sums inside its groups of 4, then over both lanes' groups
+    float before = 0.f;
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      float l[4], s = 0.f;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int t = t0 + 8 * u + 4 * g + e;
+        if (t < p.T && p.base + t >= kv0) s += log2_sigmoid(z[n][4 * u + e] + bias[n]) * p.inv_tau;
+        l[e] = s;
       }
-    }
-  }
-  float l = 0.f;
+      const float o = __shfl_xor(s, 32, 64), at = before + (g ? o : 0.f);
 #pragma unroll
-  for (int i = 0; i < kSub; ++i) {
-    const int t = t0 + wave * kSub + i;
-    if (t < p.T && p.base + t >= kv0) l += log2_sigmoid(z[i]) * p.inv_tau;
-    if (t < p.T && ch < Hd) p.cum[(static_cast<int64_t>(b) * p.T + t) * Hd + ch] = l;
+      for (int e = 0; e < 4; ++e) {
+        const int t = t0 + 8 * u + 4 * g + e;
+        if (t < p.T && ch < Hd) p.cum[(row0 + t) * Hd + ch] = at + l[e];
+      }
+      before += s + o;
+    }
+    if (g == 0) tot[wave][32 * n + c32] = before;
   }
-  tot[wave][lane] = l;
   __syncthreads();
+  const int ch = blockIdx.y * 64 + lane;
   if (wave == 0 && ch < Hd)
     p.total[(static_cast<int64_t>(b) * p.nc + blockIdx.x) * Hd + ch] = tot[0][lane] + tot[1][lane] + tot[2][lane] + tot[3][lane];
 }
@@ -409,7 +422,7 @@ __global__ __launch_bounds__(kThreads, NK > 8 || NV > 4 ? 1 : 2) void gla_output
 int gla_chunks(bool bf16, const GlaParams& p) {
   const auto al = [](const void* x) { return reinterpret_cast<uintptr_t>(x) % 16 == 0; };
   const bool ok = bf16 && p.T >= 16 && p.dim % 8 == 0 && p.vdim % 8 == 0 && p.ld % 8 == 0 && p.dim <= 256 && p.vdim <= 256 &&
-                  al(p.proj) && al(p.y) && al(p.norm_w);
+                  al(p.proj) && al(p.y) && al(p.norm_w) && al(p.a2);
   return ok ? (p.T + kC - 1) / kC : 0;
 }
 

@@ -21,7 +21,7 @@ namespace dla {
 namespace {
 
 constexpr int kTT = 64;    // tokens per tile
-constexpr int kNC = 128;   // channels per pass
+constexpr int kNC = 128;   // channels a workgroup takes, or half of them
 constexpr int kKC = 256;   // gate-block inputs staged at a time
 
 template <typename T>
@@ -54,51 +54,51 @@ __device__ __forceinline__ float conv_at(const LruParams& p, int ch, int64_t pos
   return to_f<T>(from_f<T>(s));
 }
 
-// The same for 8 channels ch .. ch + 7 and consecutive columns, bf16, TAPS taps: `row(j)` is the raw x row of
-// column col0 + j (j >= -(TAPS - 1)), pos0 the position of column col0; emits u of n columns.
-template <int TAPS, typename F, typename G>
-__device__ __forceinline__ void conv8(const LruParams& p, int ch, int64_t pos0, int n, F row, G emit) {
-  float w[8][TAPS], xb[8], cb[8], win[TAPS][8];
+// The same for V channels ch .. ch + V - 1 (V divides ch) and consecutive columns, bf16, TAPS taps: `row(j)` is the
+// raw x row of column col0 + j (j >= -(TAPS - 1)), pos0 the position of column col0; emits u of n columns.
+template <int TAPS, int V, typename F, typename G>
+__device__ __forceinline__ void conv_run(const LruParams& p, int ch, int64_t pos0, int n, F row, G emit) {
+  float w[V][TAPS], xb[V], cb[V], win[TAPS][V];
   {
     const bf16_t* src = static_cast<const bf16_t*>(p.conv_w) + static_cast<int64_t>(ch) * TAPS;
-    bf16x8 v[TAPS];
+    float v[TAPS][V];
 #pragma unroll
-    for (int i = 0; i < TAPS; ++i) v[i] = load_bf16x8(src + 8 * i);
+    for (int i = 0; i < TAPS; ++i) load_vec<bf16_t, V>(src + V * i, v[i]);
 #pragma unroll
-    for (int e = 0; e < 8; ++e)
+    for (int e = 0; e < V; ++e)
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) w[e][j] = bf2f(v[(e * TAPS + j) / 8][(e * TAPS + j) % 8]);
-    load_vec<bf16_t, 8>(static_cast<const bf16_t*>(p.bias) + p.W + ch, xb);
-    load_vec<bf16_t, 8>(static_cast<const bf16_t*>(p.conv_b) + ch, cb);
+      for (int j = 0; j < TAPS; ++j) w[e][j] = v[(e * TAPS + j) / V][(e * TAPS + j) % V];
+    load_vec<bf16_t, V>(static_cast<const bf16_t*>(p.bias) + p.W + ch, xb);
+    load_vec<bf16_t, V>(static_cast<const bf16_t*>(p.conv_b) + ch, cb);
   }
   auto fetch = [&](int j, float* o) {  // biased x of column col0 + j, zero before the start
     if (pos0 + j >= 0) {
-      load_vec<bf16_t, 8>(row(j), o);
+      load_vec<bf16_t, V>(row(j), o);
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] += xb[e];
+      for (int e = 0; e < V; ++e) o[e] += xb[e];
     } else {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) o[e] = 0.f;
+      for (int e = 0; e < V; ++e) o[e] = 0.f;
     }
   };
 #pragma unroll
   for (int j = 0; j < TAPS - 1; ++j) fetch(j - (TAPS - 1), win[j + 1]);
-#pragma unroll 2
+#pragma unroll V == 4 ? 4 : 2
   for (int t = 0; t < n; ++t) {
 #pragma unroll
     for (int j = 0; j < TAPS - 1; ++j)
 #pragma unroll
-      for (int e = 0; e < 8; ++e) win[j][e] = win[j + 1][e];
+      for (int e = 0; e < V; ++e) win[j][e] = win[j + 1][e];
     fetch(t, win[TAPS - 1]);
-    float u[8];
+    float u[V];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
+    for (int e = 0; e < V; ++e) {
       u[e] = cb[e];
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) u[e] += w[e][j] * win[j][e];
       if (pos0 + t < 0) u[e] = 0.f;
     }
-    emit(t, pack_bf16x8(u));
+    emit(t, u);
   }
 }
 
@@ -119,13 +119,13 @@ __device__ __forceinline__ typename Mma<T>::Frag gate_frag(const T* wb, int n, i
   return f;
 }
 
-// grid (nc, nb * ceil(n / (128 JG)), B), 256 threads; JG passes of 128 channels over a staged tile
-// (ONE: n <= kKC, the tile is staged once; JG > 1 only then). TAPS > 0: bf16, n % 8 == 0.
+// grid (nc, nb * ceil(n / (128 JG)), B), 256 threads, 128 JG channels (ONE: n <= kKC, a tile of tokens is
+// staged once; JG > 1 only then). TAPS > 0: bf16, n % 8 == 0.
 template <typename T, bool VEC, int TAPS, int JG, bool ONE>
-__global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
+__global__ __launch_bounds__(256, ONE ? 4 : 2) void lru_gates_kernel(LruParams p) {
   extern __shared__ __attribute__((aligned(16))) unsigned char smem[];
   using M = Mma<T>;
-  constexpr int MT = kTT / 16, NJ = kNC / 64;
+  constexpr int MT = kTT / 16, NJ = JG * kNC / 64, JA = ONE ? 1 : NJ;
   const int nblk = (p.n + kNC * JG - 1) / (kNC * JG);
   const int b = blockIdx.z, blk = blockIdx.y / nblk, c0 = (blockIdx.y % nblk) * kNC * JG;
   const int kc = min(kKC, round_up(p.n, 32)), ldu = kc + pad16<T>();
@@ -136,36 +136,33 @@ __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
   const T* Hs = static_cast<const T*>(p.hist) + static_cast<int64_t>(b) * p.taps * p.W + blk * p.n;
   const T* Wr = static_cast<const T*>(p.gates) + static_cast<int64_t>(blk) * p.n * p.n;
   const T* Wi = static_cast<const T*>(p.gates) + static_cast<int64_t>(p.nb + blk) * p.n * p.n;
-  float lam_c[JG][NJ], rb[JG][NJ], ib[JG][NJ], ca[JG][NJ], cs[JG][NJ];
-#pragma unroll
-  for (int q = 0; q < JG; ++q)
-#pragma unroll
-    for (int j = 0; j < NJ; ++j) {
-      const int ch = min(c0 + kNC * q + 16 * (wave + 4 * j) + r, p.n - 1);
-      lam_c[q][j] = -p.c * softplus(to_f<T>(static_cast<const T*>(p.lam)[blk * p.n + ch]));
-      rb[q][j] = to_f<T>(static_cast<const T*>(p.gates_b)[blk * p.n + ch]);
-      ib[q][j] = to_f<T>(static_cast<const T*>(p.gates_b)[(p.nb + blk) * p.n + ch]);
-      ca[q][j] = 1.f;
-      cs[q][j] = 0.f;
-    }
+  __shared__ float prm[3][kNC * JG], carry[2][kNC * JG];  // per channel: -c softplus(lam), gate biases; A, S so far
+  for (int i = threadIdx.x; i < kNC * JG; i += 256) {
+    const int ch = min(c0 + i, p.n - 1);
+    prm[0][i] = -p.c * softplus(to_f<T>(static_cast<const T*>(p.lam)[blk * p.n + ch]));
+    prm[1][i] = to_f<T>(static_cast<const T*>(p.gates_b)[blk * p.n + ch]);
+    prm[2][i] = to_f<T>(static_cast<const T*>(p.gates_b)[(p.nb + blk) * p.n + ch]);
+    carry[0][i] = 1.f;
+    carry[1][i] = 0.f;
+  }
   auto stage = [&](int t0, int k0) {
     if constexpr (TAPS > 0) {
-      const int ng = kc / 8, ntg = 256 / ng, per = (kTT + ntg - 1) / ntg;
-      const int k = static_cast<int>(threadIdx.x) % ng * 8, tg = threadIdx.x / ng * per;
+      constexpr int V = 4;
+      const int ng = kc / V, ntg = 256 / ng, per = (kTT + ntg - 1) / ntg;
+      const int k = static_cast<int>(threadIdx.x) % ng * V, tg = threadIdx.x / ng * per;
       const int n = min(min(per, kTT - tg), p.T - t0 - tg);  // columns of this thread that exist
-      if (tg < kTT && k0 + k < p.n && n > 0) {
+      const bool real = k0 + k < p.n;
+      if (tg < kTT && real && n > 0) {
         const int64_t col = p.base + t0 + tg;
-        conv8<TAPS>(p, blk * p.n + k0 + k, col - kv0, n,
-                    [&](int j) {
-                      return t0 + tg + j >= 0 ? X + static_cast<int64_t>(t0 + tg + j) * 2 * p.W + k0 + k
-                                              : Hs + ((col + j) % TAPS) * p.W + k0 + k;
-                    },
-                    [&](int t, bf16x8 u) { store_bf16x8(us + (tg + t) * ldu + k, u); });
+        conv_run<TAPS, V>(p, blk * p.n + k0 + k, col - kv0, n,
+                          [&](int j) {
+                            return t0 + tg + j >= 0 ? X + static_cast<int64_t>(t0 + tg + j) * 2 * p.W + k0 + k
+                                                    : Hs + ((col + j) % TAPS) * p.W + k0 + k;
+                          },
+                          [&](int t, const float* u) { store_vec<bf16_t, V>(us + (tg + t) * ldu + k, u); });
       }
-      const bf16x8 z = {0, 0, 0, 0, 0, 0, 0, 0};
-      for (int t = max(tg, tg + max(n, 0)); t < min(tg + per, kTT); ++t) store_bf16x8(us + t * ldu + k, z);
-      if (k0 + k >= p.n && tg < kTT)
-        for (int t = tg; t < min(tg + per, kTT); ++t) store_bf16x8(us + t * ldu + k, z);
+      const float z[V] = {0.f, 0.f, 0.f, 0.f};
+      for (int t = real ? tg + max(n, 0) : tg; t < min(tg + per, kTT); ++t) store_vec<bf16_t, V>(us + t * ldu + k, z);
     } else {
       for (int i = threadIdx.x; i < kTT * kc; i += 256) {
         const int t = i / kc, k = i % kc;
@@ -182,17 +179,18 @@ __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
   };
   const int t_end = min((static_cast<int>(blockIdx.x) + 1) * p.chunk, p.T);
   for (int t0 = blockIdx.x * p.chunk; t0 < t_end; t0 += kTT) {
+    if constexpr (ONE) {
+      __syncthreads();  // every wave is done with the last tile
+      stage(t0, 0);
+      __syncthreads();
+    }
+    // the wave's 16-channel tiles; when a staged tile holds all inputs (ONE), one after the other
+#pragma unroll 1
+    for (int j0 = 0; j0 < NJ; j0 += JA) {
+      f32x4 ar[JA][MT], ai[JA][MT];
+      float u[JA][MT][4];
 #pragma unroll
-    for (int q = 0; q < JG; ++q) {
-      if (ONE && q == 0) {
-        __syncthreads();  // every wave is done with the last tile
-        stage(t0, 0);
-        __syncthreads();
-      }
-      f32x4 ar[NJ][MT], ai[NJ][MT];
-      float u[NJ][MT][4];
-#pragma unroll
-      for (int j = 0; j < NJ; ++j)
+      for (int j = 0; j < JA; ++j)
 #pragma unroll
         for (int m = 0; m < MT; ++m) {
           ar[j][m] = ai[j][m] = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -206,8 +204,8 @@ __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
           __syncthreads();
         }
 #pragma unroll
-        for (int j = 0; j < NJ; ++j) {
-          const int n0 = c0 + kNC * q + 16 * (wave + 4 * j);
+        for (int j = 0; j < JA; ++j) {
+          const int n0 = c0 + 16 * (wave + 4 * (j0 + j));
           if (n0 >= p.n) continue;
 #pragma unroll 4
           for (int k = 0; k < kc; k += M::KS) {
@@ -229,9 +227,11 @@ __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
         }
       }
 #pragma unroll
-      for (int j = 0; j < NJ; ++j) {
-        const int n0 = c0 + kNC * q + 16 * (wave + 4 * j), ch = n0 + r;
-        if (n0 >= p.n) continue;
+      for (int j = 0; j < JA; ++j) {
+        const int cl = 16 * (wave + 4 * (j0 + j)) + r, ch = c0 + cl;
+        if (ch - r >= p.n) continue;
+        const float lam_c = prm[0][cl], rb = prm[1][cl], ib = prm[2][cl];
+        float ca = carry[0][cl], cs = carry[1][cl];
 #pragma unroll
         for (int m = 0; m < MT; ++m) {
           // 4 tokens of this lane: A[i], S[i] = product of decays / state since the lane's first token
@@ -241,7 +241,7 @@ __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
             const int t = t0 + 16 * m + 4 * g + i;
             float a, x;
             const float uv = ONE ? to_f<T>(us[(16 * m + 4 * g + i) * ldu + min(ch, kc - 1)]) : u[j][m][i];
-            lru_step(ar[j][m][i] + rb[q][j], ai[j][m][i] + ib[q][j], uv, lam_c[q][j], a, x);
+            lru_step(ar[j][m][i] + rb, ai[j][m][i] + ib, uv, lam_c, a, x);
             const bool real = t < p.T && p.base + t >= kv0;
             a = real ? a : 1.f;
             ps = a * ps + (real ? x : 0.f);
@@ -263,8 +263,8 @@ __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
             ea = 1.f;
             es = 0.f;
           }
-          es = ea * cs[q][j] + es;
-          ea *= ca[q][j];
+          es = ea * cs + es;
+          ea *= ca;
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
             const int t = t0 + 16 * m + 4 * g + i;
@@ -275,8 +275,12 @@ __global__ __launch_bounds__(256, 2) void lru_gates_kernel(LruParams p) {
             }
           }
           const float la = __shfl(pa, 48 + r, 64), ls = __shfl(ps, 48 + r, 64);
-          cs[q][j] = la * cs[q][j] + ls;
-          ca[q][j] *= la;
+          cs = la * cs + ls;
+          ca *= la;
+        }
+        if (g == 0) {  // (channels of this wave alone: its LDS accesses stay in order)
+          carry[0][cl] = ca;
+          carry[1][cl] = cs;
         }
       }
     }
@@ -385,12 +389,12 @@ __global__ __launch_bounds__(256) void lru_decode_kernel(LruParams p) {
         const int m = i / (kc / 8), k = i % (kc / 8) * 8, b = b0 + m;
         if (m < nr && k0 + k < p.n) {
           const int cc = blk * p.n + k0 + k;
-          conv8<TAPS>(p, cc, col - (p.kv_start ? p.kv_start[b] : 0), 1,
-                      [&](int j) {
-                        return j == 0 ? YX + static_cast<int64_t>(b) * 2 * p.W + p.W + cc
-                                      : Hs + (static_cast<int64_t>(b) * TAPS + (col + j) % TAPS) * p.W + cc;
-                      },
-                      [&](int, bf16x8 u) { store_bf16x8(us + m * ldu + k, u); });
+          conv_run<TAPS, 8>(p, cc, col - (p.kv_start ? p.kv_start[b] : 0), 1,
+                            [&](int j) {
+                              return j == 0 ? YX + static_cast<int64_t>(b) * 2 * p.W + p.W + cc
+                                            : Hs + (static_cast<int64_t>(b) * TAPS + (col + j) % TAPS) * p.W + cc;
+                            },
+                            [&](int, const float* u) { store_vec<bf16_t, 8>(us + m * ldu + k, u); });
         } else {
           store_bf16x8(us + m * ldu + k, bf16x8{0, 0, 0, 0, 0, 0, 0, 0});
         }
@@ -446,7 +450,7 @@ __global__ __launch_bounds__(256) void lru_decode_kernel(LruParams p) {
   static_cast<T*>(p.out)[at] = from_f<T>(S * gelu_tanh(to_f<T>(y0) + yb));
 }
 
-// passes of 128 channels per workgroup
+// multiples of 128 channels per workgroup
 int lru_passes(const LruParams& p) { return p.n > kNC && p.n <= kKC ? 2 : 1; }
 
 template <typename K>

@@ -588,6 +588,19 @@ def test_meta_build_matches_and_presets():
         assert c.name == name and c.num_params() > 5e8 and c.flops_per_token(2048) > 1e9
 
 
+def test_serving_bench_peers():
+    """The models measured beside a size have its layer count, width, heads and feed-forward parameters."""
+    from distributed_llm_alignment_amd.eval import serve_bench
+
+    for name in serve_bench.SIZES["zenevik"]:
+        cfg = get_config(name)
+        peers = serve_bench.peers(cfg)
+        assert set(peers) == {"peer", "peer_attention"}
+        for p in peers.values():
+            assert p.num_layers == cfg.num_layers and p.hidden_size == cfg.hidden_size and p.vocab_size == cfg.vocab_size
+            assert 0.8 < p.num_params() / cfg.num_params() < 1.2
+
+
 def test_bad_configs_are_refused():
     for edit in (lambda c: c["layers"][0].update(type="retention"),
                  lambda c: c["layers"][0]["mixer"].update(blocks=7),
